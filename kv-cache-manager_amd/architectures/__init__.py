@@ -4,3 +4,4 @@ from . import kasuvik  # noqa: F401
 from . import furapel  # noqa: F401
 from . import fisesun  # noqa: F401
 from . import betirax  # noqa: F401
+from . import vugotar  # noqa: F401

@@ -20,12 +20,14 @@ _KIND_NAMES = {"full": FULL_KV, "window": WINDOW_KV, "state": STATE}
 @dataclass(frozen=True)
 class CacheGroupSpec:
     """kind: "full" (every key kept), "window" (a query at p sees keys t with p - t < window, and the first
-    ``keep_first`` tokens of its sequence: their pages stay when the window has passed them)
+    ``keep_first`` tokens of its sequence: their pages stay when the window has passed them; with ``chunk`` > 0 it sees
+    the keys of its own chunk, t // chunk == p // chunk, and a chunk's pages go back when the next begins)
     or "state" (fixed-size per-request state, no pages)."""
     kind: str = "full"
     window: int = 0
     num_blocks: int = 0
     keep_first: int = 0
+    chunk: int = 0
 
 
 def _i32(a):
@@ -158,6 +160,8 @@ class HostCore:
         for g, spec in enumerate(self.groups):
             if spec.keep_first:
                 check(self._lib.kvcm_core_keep_first(self._h, g, spec.keep_first))
+            if spec.chunk:
+                check(self._lib.kvcm_core_chunk(self._h, g, spec.chunk))
         self.policy = policy
         self.block_size = block_size
         self.max_seq_len = max_seq_len

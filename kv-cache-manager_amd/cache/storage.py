@@ -70,9 +70,11 @@ class KVStorage:
 
     def bytes_read(self, context: int) -> int:
         """Bytes a request with ``context`` tokens has a step read from this group: the keys and values of
-        every layer, of the window's tokens where there is a window (and the pooled entries before it)."""
+        every layer, of the window's (or the last token's chunk's) tokens where there is one (and the pooled entries before it)."""
         n = self.need
         tokens = min(context, n.window) if n.window > 0 else context
+        if n.chunk > 0 and context > 0:
+            tokens = min(tokens, (context - 1) % n.chunk + 1)
         token_bytes = self.num_layers * n.num_kv_heads * (n.head_dim + self.value_dim) * self._k.element_size()
         pooled = 0
         if n.pool > 0 and n.window > 0 and context > n.window:

@@ -5,10 +5,12 @@
 //   row at position i sees   tokens j with 0 <= i - j < window
 //                            blocks b with b*P + P - 1 <= i - window   (mean key, mean value of its P tokens)
 //                            tokens j < keep_first (the sequence's first tokens stay visible beyond the window)
+//                            with a chunk size instead of a window: tokens j <= i with j / chunk == i / chunk
 //   and all of them share one softmax; score = (q . k) * scale_h with a factor per query head, and with a cap c > 0
 //   score <- c tanh(score / c); then, with a slope per query head, score <- score - slope_h * (i - j) for token j (a bias
 //   that grows with the distance; not offered together with pooled blocks, which have no one distance).  The output may be
-//   multiplied element by element with sigmoid(gate) (32-bit gate logits of the output's shape) before it is stored.
+//   multiplied element by element with sigmoid(gate) (32-bit gate logits of the output's shape) before it is stored, and by a
+//   constant factor.  With a sink, one is added to the softmax's denominator: a key of score 0 that has no value.
 //
 // Pages: keys [pages, kv_heads, B, d], values transposed [pages, kv_heads, dv, B] (as the other
 // attentions of this library keep them).  Pooled entries are 32-bit and live with the page that holds
@@ -265,7 +267,7 @@ __global__ void __launch_bounds__(kWpWaves* kWave)
                                  const int* __restrict__ ctx_lens, const float* __restrict__ head_scale,
                                  const float* __restrict__ dist_slope, const float* __restrict__ gate, int ldg,
                                  int nh, int nkv, int d, int dv, int B, float scale, int window, int P, int E, int keep_first,
-                                 float softcap) {
+                                 float softcap, int chunk, int sink, float out_scale) {
   extern __shared__ float lds[];      // [d] q * scale * head_scale[h]; [waves][64] probabilities; [waves][dv + 2] results
   constexpr int N = RowPiece<T>::N, COLS = kWpMaxValueDim / kWave;
   const int wave = threadIdx.x / kWave, lane = threadIdx.x % kWave;
@@ -286,7 +288,7 @@ __global__ void __launch_bounds__(kWpWaves* kWave)
     return;
   }
   const int* table = tables + size_t(row_seq[row]) * table_stride;
-  const int first = (window > 0 && ctx > window) ? ctx - window : 0;
+  const int first = chunk > 0 ? (ctx - 1) / chunk * chunk : (window > 0 && ctx > window) ? ctx - window : 0;
   const int blocks = (P > 0 && window > 0 && ctx - window >= P) ? (ctx - window) / P : 0;      // those that end at or before ctx - 1 - window
   const int block_chunks = (blocks + kWave - 1) / kWave;
   // tokens at the sequence's start that stay visible beyond the window: those of them that lie before the window's
@@ -408,10 +410,10 @@ __global__ void __launch_bounds__(kWpWaves* kWave)
     mine[dv + 1] = l;
   }
   __syncthreads();
-  float mm = -INFINITY;
+  float mm = sink ? 0.f : -INFINITY;
 #pragma unroll
   for (int w = 0; w < kWpWaves; ++w) mm = fmaxf(mm, merge[w * (dv + 2) + dv]);
-  float wgt[kWpWaves], ll = 0.f;
+  float wgt[kWpWaves], ll = sink ? expf(-mm) : 0.f;
 #pragma unroll
   for (int w = 0; w < kWpWaves; ++w) {
     const float mw = merge[w * (dv + 2) + dv];
@@ -422,7 +424,7 @@ __global__ void __launch_bounds__(kWpWaves* kWave)
     float acc = 0.f;
 #pragma unroll
     for (int w = 0; w < kWpWaves; ++w) acc = fmaf(merge[w * (dv + 2) + cc], wgt[w], acc);
-    float res = acc / ll;
+    float res = acc / ll * out_scale;
     if (gate) res *= 1.0f / (1.0f + expf(-gate[size_t(row) * ldg + size_t(head) * dv + cc]));      // a gate per element of the output
     store_f(orow + cc, res);
   }
@@ -526,7 +528,7 @@ int kvcm_attention_window_pool(const void* q, int dtype, int ldq, void* out, int
                                const float* pk, const float* pv, const int* tables, int table_stride, const int* row_seq,
                                const int* ctx_lens, const float* head_scale, const float* dist_slope, const float* gate, int ldg,
                                int T, int nh, int nkv, int d, int dv, int B, float scale, int window, int P, int E, int keep_first,
-                               float softcap, hipStream_t s) {
+                               float softcap, int chunk, int sink, float out_scale, hipStream_t s) {
   if (T == 0) return 0;
   KVCM_REQUIRE(T > 0 && nh > 0 && nkv > 0 && B > 0 && d > 0, "attention_window_pool: bad sizes T=%d heads=%d kv_heads=%d", T, nh, nkv);
   KVCM_REQUIRE(nh % nkv == 0, "attention_window_pool: %d query heads are not a multiple of %d kv heads", nh, nkv);
@@ -538,6 +540,8 @@ int kvcm_attention_window_pool(const void* q, int dtype, int ldq, void* out, int
   KVCM_REQUIRE(keep_first >= 0 && softcap >= 0.f, "attention_window_pool: negative count of kept tokens or score cap");
   KVCM_REQUIRE(!dist_slope || P == 0, "attention_window_pool: a distance bias beside pooled blocks is not supported");
   KVCM_REQUIRE(!gate || ldg >= nh * dv, "attention_window_pool: the gate's rows are too short");
+  KVCM_REQUIRE(chunk >= 0 && (chunk == 0 || (window == 0 && P == 0 && keep_first == 0)),
+               "attention_window_pool: a chunk beside a window, pooled blocks or kept first tokens is not supported");
   const long long blocks = static_cast<long long>(T) * nh;
   KVCM_REQUIRE(blocks < (1ll << 31), "attention_window_pool: too many rows");
   const size_t lds = sizeof(float) * (d + kWpWaves * kWave + kWpWaves * (dv + 2));
@@ -545,12 +549,12 @@ int kvcm_attention_window_pool(const void* q, int dtype, int ldq, void* out, int
     attention_window_pool_kernel<float><<<static_cast<unsigned>(blocks), kWpWaves * kWave, lds, s>>>(
         static_cast<const float*>(q), ldq, static_cast<float*>(out), ldo, static_cast<const float*>(kcache),
         static_cast<const float*>(vcache), pk, pv, tables, table_stride, row_seq, ctx_lens, head_scale, dist_slope, gate,
-        ldg, nh, nkv, d, dv, B, scale, window, P, E, keep_first, softcap);
+        ldg, nh, nkv, d, dv, B, scale, window, P, E, keep_first, softcap, chunk, sink, out_scale);
   else if (dtype == kBF16)
     attention_window_pool_kernel<bf16_t><<<static_cast<unsigned>(blocks), kWpWaves * kWave, lds, s>>>(
         static_cast<const bf16_t*>(q), ldq, static_cast<bf16_t*>(out), ldo, static_cast<const bf16_t*>(kcache),
         static_cast<const bf16_t*>(vcache), pk, pv, tables, table_stride, row_seq, ctx_lens, head_scale, dist_slope, gate,
-        ldg, nh, nkv, d, dv, B, scale, window, P, E, keep_first, softcap);
+        ldg, nh, nkv, d, dv, B, scale, window, P, E, keep_first, softcap, chunk, sink, out_scale);
   else KVCM_REQUIRE(false, "attention_window_pool: unknown dtype %d", dtype);
   return launch_status("attention_window_pool");
 }

@@ -10,7 +10,8 @@
 // keep_first tokens of a sequence may stay visible beyond the window (chunks of their own, from token 0), and the
 // scores may be capped, score <- c tanh(score / c), and a bias that grows with the distance may be taken off them,
 // score <- score - slope_h * (i - j) with a slope per query head (tokens only: not beside pooled blocks); the output may be
-// multiplied element by element with sigmoid(gate) before it is stored.
+// multiplied element by element with sigmoid(gate) before it is stored, and by a constant factor.  With a chunk size in the
+// window's place a row sees its own chunk of positions only; with a sink, one is added to the softmax's denominator.
 // bfloat16 storage only; sizes d and dv in multiples of 8, pages whose size is a multiple of 8 and divides 64.
 #include <cfloat>
 
@@ -39,7 +40,7 @@ __global__ void __launch_bounds__(256)
                                        const int* __restrict__ seq_start, const float* __restrict__ head_scale,
                                        const float* __restrict__ dist_slope, const float* __restrict__ gate, int ldg, int tiles_per_seq,
                                        int nh, int nkv, int d, int dv, int B, float scale, int window, int P, int E,
-                                       int keep_first, float softcap) {
+                                       int keep_first, float softcap, int chunk, int sink, float out_scale) {
   constexpr int KP = DP + 8, KS = DP / 32, DVP = DVT * 16;
   __shared__ __attribute__((aligned(16))) uint16_t Ks[kChunk][KP];
   __shared__ __attribute__((aligned(16))) uint16_t Vt[DVP][kVtPitch];
@@ -76,13 +77,14 @@ __global__ void __launch_bounds__(256)
     }
   }
   // the four rows whose scores this lane holds: 4 * quad + i of the wave's 16
-  int pos[4], seen_blocks[4];
+  int pos[4], seen_blocks[4], lo_pos[4];      // lo_pos: the first token of the row's window or chunk
   float m[4], lsum[4];
 #pragma unroll
   for (int i = 0; i < 4; ++i) {
     const int row = wave * 16 + quad * 4 + i;
     pos[i] = row < nrows ? p0 + row : -1;
     seen_blocks[i] = (P > 0 && window > 0 && pos[i] + 1 > window) ? (pos[i] + 1 - window) / P : 0;
+    lo_pos[i] = chunk > 0 ? pos[i] / chunk * chunk : window > 0 ? pos[i] - window + 1 : 0;
     m[i] = kMasked;
     lsum[i] = 0.f;
   }
@@ -91,7 +93,7 @@ __global__ void __launch_bounds__(256)
   for (int vt = 0; vt < DVT; ++vt) o[vt] = f32x4{0.f, 0.f, 0.f, 0.f};
 
   const int blocks = (P > 0 && window > 0 && p_last + 1 > window) ? (p_last + 1 - window) / P : 0;      // of the tile's last row
-  const int t_lo = (window > 0 && p0 + 1 > window) ? p0 + 1 - window : 0;
+  const int t_lo = chunk > 0 ? p0 / chunk * chunk : (window > 0 && p0 + 1 > window) ? p0 + 1 - window : 0;
   const int block_chunks = (blocks + kChunk - 1) / kChunk;
   // the sequence's first tokens that stay visible beyond the window: those before the tile's first seen token get chunks
   // of their own, from token 0, between the blocks and the window (every row of the tile sees all of them)
@@ -202,7 +204,7 @@ __global__ void __launch_bounds__(256)
         const int key = c0 + ct * 16 + col;
         vis[ct] = pooled ? key < seen_blocks[i]
                   : early ? (key < kept && pos[i] >= 0)
-                          : (key >= t_lo && key <= pos[i] && (window == 0 || key > pos[i] - window || key < keep_first));
+                          : (key >= t_lo && key <= pos[i] && (key >= lo_pos[i] || key < keep_first));
         float sv = sc[ct][i] * f;
         if (softcap > 0.f) sv = cap2 * tanhf(sv);
         if (dist_slope) sv = fmaf(-slope2, float(pos[i] - key), sv);
@@ -241,10 +243,16 @@ __global__ void __launch_bounds__(256)
   }
 #pragma unroll
   for (int i = 0; i < 4; ++i) {
-    const float l = group_sum<16>(lsum[i]);
+    float l = group_sum<16>(lsum[i]), factor = out_scale;
+    if (sink) {      // a score of 0 joins the denominator (scores are in units of log 2 here too)
+      const float m_all = fmaxf(m[i], 0.f);
+      const float keep = __builtin_amdgcn_exp2f(m[i] - m_all);
+      l = l * keep + __builtin_amdgcn_exp2f(-m_all);
+      factor *= keep;
+    }
     const int row = wave * 16 + quad * 4 + i;
     if (row < nrows) {
-      const float inv = 1.0f / l;
+      const float inv = factor / l;
 #pragma unroll
       for (int vt = 0; vt < DVT; ++vt) {
         const int cc = vt * 16 + col;
@@ -262,11 +270,12 @@ template <int DP>
 int launch_tiles(int dvt, dim3 grid, hipStream_t s, const uint16_t* q, int ldq, uint16_t* out, int ldo, const uint16_t* kc,
                  const uint16_t* vc, const float* pk, const float* pv, const int* tables, int table_stride, const int* run_start,
                  const int* seq_start, const float* head_scale, const float* dist_slope, const float* gate, int ldg, int tiles_per_seq,
-                 int nh, int nkv, int d, int dv, int B, float scale, int window, int P, int E, int keep_first, float softcap) {
+                 int nh, int nkv, int d, int dv, int B, float scale, int window, int P, int E, int keep_first, float softcap,
+                 int chunk, int sink, float out_scale) {
 #define KVCM_TILES(DVT)                                                                                                     \
   attention_window_pool_tiles_kernel<DP, DVT><<<grid, 256, 0, s>>>(q, ldq, out, ldo, kc, vc, pk, pv, tables, table_stride,   \
                                                                    run_start, seq_start, head_scale, dist_slope, gate, ldg, tiles_per_seq, \
-                                                                   nh, nkv, d, dv, B, scale, window, P, E, keep_first, softcap)
+                                                                   nh, nkv, d, dv, B, scale, window, P, E, keep_first, softcap, chunk, sink, out_scale)
   if (dvt <= 2) KVCM_TILES(2);
   else if (dvt <= 4) KVCM_TILES(4);
   else if (dvt <= 8) KVCM_TILES(8);
@@ -290,7 +299,7 @@ int kvcm_attention_window_pool_tiles(const void* q, int ldq, void* out, int ldo,
                                      const float* pk, const float* pv, const int* tables, int table_stride,
                                      const int* run_start, const int* seq_start, const float* head_scale, const float* dist_slope,
                                      const float* gate, int ldg, int S, int max_run, int nh, int nkv, int d, int dv, int B, float scale, int window, int P,
-                                     int E, int keep_first, float softcap, hipStream_t s) {
+                                     int E, int keep_first, float softcap, int chunk, int sink, float out_scale, hipStream_t s) {
   if (S == 0 || max_run == 0) return 0;
   KVCM_REQUIRE(S > 0 && max_run > 0 && nh > 0 && nkv > 0 && nh % nkv == 0, "attention_window_pool_tiles: bad sizes");
   KVCM_REQUIRE(kvcm_attention_window_pool_tiles_supported(d, dv, B),
@@ -303,6 +312,8 @@ int kvcm_attention_window_pool_tiles(const void* q, int ldq, void* out, int ldo,
   KVCM_REQUIRE(keep_first >= 0 && softcap >= 0.f, "attention_window_pool_tiles: negative count of kept tokens or score cap");
   KVCM_REQUIRE(!dist_slope || P == 0, "attention_window_pool_tiles: a distance bias beside pooled blocks is not supported");
   KVCM_REQUIRE(!gate || ldg >= nh * dv, "attention_window_pool_tiles: the gate's rows are too short");
+  KVCM_REQUIRE(chunk >= 0 && (chunk == 0 || (window == 0 && P == 0 && keep_first == 0)),
+               "attention_window_pool_tiles: a chunk beside a window, pooled blocks or kept first tokens is not supported");
   const int tiles_per_seq = (max_run + kTileRows - 1) / kTileRows;
   KVCM_REQUIRE(static_cast<long long>(S) * tiles_per_seq < (1ll << 31) && nh <= 65535, "attention_window_pool_tiles: too many rows");
   const dim3 grid(S * tiles_per_seq, nh);
@@ -313,12 +324,12 @@ int kvcm_attention_window_pool_tiles(const void* q, int ldq, void* out, int ldo,
   const uint16_t* vc = static_cast<const uint16_t*>(vcache);
   if (d <= 32)
     return launch_tiles<32>(dvt, grid, s, qq, ldq, oo, ldo, kc, vc, pk, pv, tables, table_stride, run_start, seq_start, head_scale,
-                            dist_slope, gate, ldg, tiles_per_seq, nh, nkv, d, dv, B, scale, window, P, E, keep_first, softcap);
+                            dist_slope, gate, ldg, tiles_per_seq, nh, nkv, d, dv, B, scale, window, P, E, keep_first, softcap, chunk, sink, out_scale);
   if (d <= 64)
     return launch_tiles<64>(dvt, grid, s, qq, ldq, oo, ldo, kc, vc, pk, pv, tables, table_stride, run_start, seq_start, head_scale,
-                            dist_slope, gate, ldg, tiles_per_seq, nh, nkv, d, dv, B, scale, window, P, E, keep_first, softcap);
+                            dist_slope, gate, ldg, tiles_per_seq, nh, nkv, d, dv, B, scale, window, P, E, keep_first, softcap, chunk, sink, out_scale);
   return launch_tiles<128>(dvt, grid, s, qq, ldq, oo, ldo, kc, vc, pk, pv, tables, table_stride, run_start, seq_start, head_scale,
-                           dist_slope, gate, ldg, tiles_per_seq, nh, nkv, d, dv, B, scale, window, P, E, keep_first, softcap);
+                           dist_slope, gate, ldg, tiles_per_seq, nh, nkv, d, dv, B, scale, window, P, E, keep_first, softcap, chunk, sink, out_scale);
 }
 
 }  // extern "C"

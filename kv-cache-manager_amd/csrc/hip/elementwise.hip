@@ -446,11 +446,17 @@ __global__ void embed_scaled_kernel(const int* __restrict__ ids, const TW* __res
 // (0.5 z (1 + tanh(sqrt(2/pi) (z + 0.044715 z^3)))).  Computed in 32-bit, rounded once.
 template <class TO>
 __global__ void __launch_bounds__(256)
-    gated_act_kernel(const float* __restrict__ gu, int ld, TO* __restrict__ out, int ldo, int I, int act) {
+    gated_act_kernel(const float* __restrict__ gu, int ld, const float* __restrict__ bias, const float* __restrict__ row_gate, int ldr,
+                     TO* __restrict__ out, int ldo, int I, int act) {
   const int t = blockIdx.y;
   const int i = blockIdx.x * blockDim.x + threadIdx.x;
   if (i >= I) return;
-  const float g = gu[size_t(t) * ld + i], u = gu[size_t(t) * ld + I + i];
+  float g = gu[size_t(t) * ld + i], u = gu[size_t(t) * ld + I + i];
+  if (bias) {      // [2I]: the gate's, then the other projection's
+    g += bias[i];
+    u += bias[I + i];
+  }
+  if (row_gate) u *= 1.0f / (1.0f + expf(-row_gate[size_t(t) * ldr]));      // one gate logit per row
   float a;
   if (act == 1) a = fmaxf(g, 0.f);
   else if (act == 2) a = 0.5f * g * (1.0f + tanhf(0.7978845608028654f * (g + 0.044715f * g * g * g)));
@@ -496,14 +502,14 @@ int kvcm_embed_scaled(const int* ids, const void* table, int table_dtype, float*
   return launch_status("embed_scaled");
 }
 
-int kvcm_gated_act(const float* gate_up, int ld, void* out, int out_dtype, int ldo, int T, int I, int act, hipStream_t s) {
+int kvcm_gated_act(const float* gate_up, int ld, const float* bias, const float* row_gate, int ldr, void* out, int out_dtype, int ldo, int T, int I, int act, hipStream_t s) {
   if (T == 0) return 0;
   KVCM_REQUIRE(T > 0 && I > 0 && ld >= 2 * I && ldo >= I, "gated_act: bad sizes T=%d I=%d", T, I);
   KVCM_REQUIRE(T <= 65535, "gated_act: too many rows for one launch (%d)", T);
   KVCM_REQUIRE(act >= 0 && act <= 2, "gated_act: unknown activation %d (0 silu, 1 relu, 2 gelu_tanh)", act);
   const dim3 grid((I + 255) / 256, T);
-  if (out_dtype == kF32) gated_act_kernel<float><<<grid, 256, 0, s>>>(gate_up, ld, static_cast<float*>(out), ldo, I, act);
-  else if (out_dtype == kBF16) gated_act_kernel<bf16_t><<<grid, 256, 0, s>>>(gate_up, ld, static_cast<bf16_t*>(out), ldo, I, act);
+  if (out_dtype == kF32) gated_act_kernel<float><<<grid, 256, 0, s>>>(gate_up, ld, bias, row_gate, ldr, static_cast<float*>(out), ldo, I, act);
+  else if (out_dtype == kBF16) gated_act_kernel<bf16_t><<<grid, 256, 0, s>>>(gate_up, ld, bias, row_gate, ldr, static_cast<bf16_t*>(out), ldo, I, act);
   else KVCM_REQUIRE(false, "gated_act: unknown output dtype %d", out_dtype);
   return launch_status("gated_act");
 }

@@ -149,14 +149,14 @@ int kvcm_probe_phases(const void* weights, const long long* phase_bytes, int pha
 // (elementwise.hip) the embedding times a factor; act(gate) * up with act 0 silu, 1 relu, 2 gelu by tanh
 int kvcm_embed_scaled(const int* ids, const void* table, int table_dtype, float* x, int T, int H, int V, float factor,
                       hipStream_t s);
-int kvcm_gated_act(const float* gate_up, int ld, void* out, int out_dtype, int ldo, int T, int I, int act, hipStream_t s);
+int kvcm_gated_act(const float* gate_up, int ld, const float* bias, const float* row_gate, int ldr, void* out, int out_dtype, int ldo, int T, int I, int act, hipStream_t s);
 // (norm_chain.hip) 32-bit RMS norms chained along a row: two branches combined, normed, added to the stream, the
 // stream normed again; the norm of every head with a weight and a sigmoid gate
 int kvcm_rmsnorm_chain(float* x, const float* a, int a_splits, const float* b, int b_splits, long long split_stride,
                        const float* wa, const float* wb, float combine, const float* w_post, const int* rows,
                        const float* w_pre, void* out, int out_dtype, int R, int H, float eps, hipStream_t s);
 int kvcm_head_norm_gate(const float* o, int ldo, const float* g, int ldg, const float* w, void* out, int out_dtype,
-                        int ldout, int T, int heads, int d, float eps, hipStream_t s);
+                        int ldout, int T, int heads, int d, float eps, int gate_silu, hipStream_t s);
 // (short_conv.hip) a short causal convolution per channel over packed runs, its last inputs kept per sequence
 int kvcm_short_conv(const float* in, int ld_in, const float* bias_in, const float* w, const float* bias_out,
                     float* state, void* out, int out_dtype, int ld_out, const int* row_seq, const int* positions,
@@ -179,7 +179,7 @@ int kvcm_attention_window_pool(const void* q, int dtype, int ldq, void* out, int
                                const float* pk, const float* pv, const int* tables, int table_stride, const int* row_seq,
                                const int* ctx_lens, const float* head_scale, const float* dist_slope, const float* gate, int ldg,
                                int T, int nh, int nkv, int d, int dv, int B, float scale, int window, int P, int E, int keep_first,
-                               float softcap, hipStream_t s);
+                               float softcap, int chunk, int sink, float out_scale, hipStream_t s);
 // as rotate_store, after q and k were divided by the root mean square of their whole stretch (times a weight) and v was
 // blended with another layer's values of the same row
 int kvcm_norm_rotate_store(const float* src, int ld, const float* wq, const float* wk, float eps, const float* v_other, int ldvo,
@@ -192,7 +192,7 @@ int kvcm_attention_window_pool_tiles(const void* q, int ldq, void* out, int ldo,
                                      const float* pk, const float* pv, const int* tables, int table_stride,
                                      const int* run_start, const int* seq_start, const float* head_scale, const float* dist_slope,
                                      const float* gate, int ldg, int S, int max_run, int nh, int nkv, int d, int dv, int B, float scale, int window, int P,
-                                     int E, int keep_first, float softcap, hipStream_t s);
+                                     int E, int keep_first, float softcap, int chunk, int sink, float out_scale, hipStream_t s);
 // (selective_scan.hip, delta_rule.hip) recurrences with a 32-bit state per sequence
 int kvcm_selective_scan(const void* x, int dtype, int ldx, const float* dt_lin, int lddt, const float* dt_bias,
                         const float* bc, int ldbc, int off_b, int off_c, const float* a_log, const float* dskip,
@@ -224,7 +224,7 @@ int kvcm_rms_groups(float* x, int ld, int col0, int size, int groups, const floa
 int kvcm_layernorm_post(float* x, const float* a, int a_splits, long long split_stride, const float* bias, float alpha,
                         const float* weight, const int* rows, void* out, int out_dtype, int R, int H, float eps, hipStream_t s);
 int kvcm_head_norm_store(const float* src, int ld, const float* bias, const float* wq, const float* wk, float eps,
-                         const int* positions, float temp_coef, int temp_every, int values_are_keys, const int* slots, void* q_out,
+                         int plain_norm, const float* cos_sin, int rot, int halves, const int* positions, float temp_coef, int temp_every, int values_are_keys, const int* slots, void* q_out,
                          int dtype, int ldq, void* kcache, void* vcache, int T, int nh, int nkv, int d, int dv, int B, hipStream_t s);
 // (gemm_heads.hip) one small product per head in one launch, with an optional sigmoid gate per element
 int kvcm_gemm_heads(const void* X, int in_dtype, int ldx, const void* W, void* Y, int out_dtype, int ldy, const float* gate,
@@ -232,6 +232,19 @@ int kvcm_gemm_heads(const void* X, int in_dtype, int ldx, const void* W, void* Y
 // (elementwise.hip) an activation without a gate on 32-bit rows
 int kvcm_act_rows(const float* in, int ld, int splits, long long split_stride, void* out, int out_dtype, int ldo, int T, int I,
                   int act, hipStream_t s);
+// (stream_terms.hip) layers whose sublayers all read one normed copy of the stream: their outputs added with a factor each, and
+// the next norm, in one launch; a gate before a norm over groups of columns
+int kvcm_stream_terms(float* x, const float* a, int a_splits, float a_factor, const float* b, int b_splits, float b_factor,
+                      const float* c, int c_splits, float c_factor, long long split_stride, const float* bias, const float* again,
+                      const int* rows, const float* w, void* out, int out_dtype, int R, int H, float eps, hipStream_t s);
+int kvcm_group_norm_gate(const float* y, int ldy, const float* z, int ldz, const float* w, void* out, int out_dtype, int ldo, int T,
+                         int groups, int size, float eps, hipStream_t s);
+// (gated_state.hip) the gated delta rule (delta 1) and the state-space recurrence with one decay per head (delta 0)
+long long kvcm_gated_state_carry_floats(int rows, int S, int heads, int dk, int dv, int delta, int piece);
+int kvcm_gated_state(const float* q, int ldq, const float* k, int ldk, const float* v, int ldv, const float* a, int lda, const float* b,
+                     int ldb, const float* dt_bias, const float* a_log, const float* d_skip, int delta, float* o, int ldo, float* state,
+                     const int* run_start, const int* seq_start, const int* state_slots, int S, int heads, int groups, int dk, int dv,
+                     int T, int piece, int max_run, float* carry, long long carry_floats, hipStream_t s);
 // (mlstm.hip) a matrix memory with exponential gates, walked token by token
 int kvcm_mlstm_scan(const float* q, int ldq, const float* k, int ldk, const float* v, int ldv, const float* ig, int ldi,
                     const float* fg, int ldf, const float* i_bias, const float* f_bias, float cap, float q_scale, float* coef,
@@ -239,7 +252,7 @@ int kvcm_mlstm_scan(const float* q, int ldq, const float* k, int ldk, const floa
                     const int* seq_start, const int* state_slots, int S, int heads, int dk, int dv, int T, int max_run,
                     hipStream_t s);
 // (moe.hip) a routed feed-forward: the choice of experts, and the experts' two products a row at a time
-int kvcm_moe_route(const float* logits, int ld, int splits, long long split_stride, int E, int top, int over_chosen, int* chosen,
+int kvcm_moe_route(const float* logits, int ld, int splits, long long split_stride, int E, int top, int over_chosen, float factor, int* chosen,
                    float* weight, int T, hipStream_t s);
 int kvcm_moe_table_route(const int* tokens, const int* table, int vocab, int ld, int top, int* chosen, float* weight, int T,
                          hipStream_t s);

@@ -3,7 +3,7 @@
 //
 //   moe_route      32-bit router logits [T, E] -> chosen[T, top] (expert numbers, best first; equal scores: the lower
 //                  number) and weight[T, top]: their softmax scores over all E, or (over_chosen) the softmax over the
-//                  chosen logits alone, which add up to one.  One wave per row.
+//                  chosen logits alone, which add up to one; times a constant factor.  One wave per row.
 //   moe_table_route  chosen[T, top] = table[token of the row, :] (a table of expert numbers per token id), weight = 1 / top
 //   moe_up         act[T, top, F] = a(W_up[e] h) for each row's chosen experts, a = square of relu, rounded to the
 //                  compute dtype; or, gated, act = silu(W_gate[e] h) * (W_up[e] h) with the two matrices of an expert
@@ -27,7 +27,7 @@ constexpr int kMoeMaxExperts = 1024;      // a row's logits are kept in LDS whil
 
 __global__ void __launch_bounds__(256)
     moe_route_kernel(const float* __restrict__ logits, int ld, int splits, size_t split_stride, int E, int top, int over_chosen,
-                     int* __restrict__ chosen, float* __restrict__ weight, int T) {
+                     float factor, int* __restrict__ chosen, float* __restrict__ weight, int T) {
   // up to 64 experts a lane group: the row's logits are formed once (a router product that was split along K arrives as
   // slices, which are added here in their order) and kept in LDS
   __shared__ float zs[256 / kWave][kMoeMaxExperts];
@@ -68,13 +68,13 @@ __global__ void __launch_bounds__(256)
     picked[s] = expf(best - mx);      // the first pick is the largest logit: exp(0)
     if (lane == 0) {
       chosen[size_t(row) * top + s] = at;
-      if (!over_chosen) weight[size_t(row) * top + s] = picked[s] * inv;
+      if (!over_chosen) weight[size_t(row) * top + s] = picked[s] * inv * factor;
     }
   }
   if (over_chosen && lane == 0) {
     float among = 0.f;
     for (int s = 0; s < top; ++s) among += picked[s];
-    const float inv_among = 1.0f / among;
+    const float inv_among = factor / among;
     for (int s = 0; s < top; ++s) weight[size_t(row) * top + s] = picked[s] * inv_among;
   }
 }
@@ -230,14 +230,14 @@ using namespace kvcm;
 
 extern "C" {
 
-int kvcm_moe_route(const float* logits, int ld, int splits, long long split_stride, int E, int top, int over_chosen, int* chosen,
+int kvcm_moe_route(const float* logits, int ld, int splits, long long split_stride, int E, int top, int over_chosen, float factor, int* chosen,
                    float* weight, int T, hipStream_t s) {
   if (T == 0) return 0;
   KVCM_REQUIRE(T > 0 && E > 0 && top > 0 && top <= E && ld >= E, "moe_route: bad sizes T=%d experts=%d top=%d", T, E, top);
   KVCM_REQUIRE(top <= kMoeMaxTop, "moe_route: %d experts a row are not supported (up to %d)", top, kMoeMaxTop);
   KVCM_REQUIRE(E <= kMoeMaxExperts, "moe_route: %d experts are not supported (up to %d)", E, kMoeMaxExperts);
   KVCM_REQUIRE(splits >= 1 && split_stride >= 0, "moe_route: the logits have at least one slice");
-  moe_route_kernel<<<(T + 3) / 4, 256, 0, s>>>(logits, ld, splits, static_cast<size_t>(split_stride), E, top, over_chosen, chosen, weight, T);
+  moe_route_kernel<<<(T + 3) / 4, 256, 0, s>>>(logits, ld, splits, static_cast<size_t>(split_stride), E, top, over_chosen, factor, chosen, weight, T);
   return launch_status("moe_route");
 }
 

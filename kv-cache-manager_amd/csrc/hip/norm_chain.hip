@@ -194,13 +194,13 @@ __global__ void __launch_bounds__(kChainThreads)
   }
 }
 
-// out[r, h, :] = n(o[r, h, :]) * w[h, :] * sigmoid(g[r, h, :]): the norm of every head on its own, a
+// out[r, h, :] = n(o[r, h, :]) * w[h, :] * act(g[r, h, :]), act = sigmoid or silu: the norm of every head on its own, a
 // plain weight over all heads, and a gate.  One wave per (row, head).
 template <class TO>
 __global__ void __launch_bounds__(256)
     head_norm_gate_kernel(const float* __restrict__ o, int ldo, const float* __restrict__ g, int ldg,
                           const float* __restrict__ w, TO* __restrict__ out, int ldout, long long items, int heads,
-                          int d, float eps) {
+                          int d, float eps, int gate_silu) {
   const long long item = static_cast<long long>(blockIdx.x) * (256 / kWave) + threadIdx.x / kWave;
   if (item >= items) return;
   const int lane = threadIdx.x % kWave;
@@ -213,7 +213,8 @@ __global__ void __launch_bounds__(256)
   const float inv = 1.0f / sqrtf(ss / float(d) + eps);
   TO* dst = out + size_t(row) * ldout + size_t(head) * d;
   for (int i = lane; i < d; i += kWave) {
-    const float gate = 1.0f / (1.0f + expf(-grow[i]));
+    const float gl = grow[i];
+    const float gate = (gate_silu ? gl : 1.0f) / (1.0f + expf(-gl));
     store_f(dst + i, orow[i] * inv * w[size_t(head) * d + i] * gate);
   }
 }
@@ -262,7 +263,7 @@ int kvcm_rmsnorm_chain(float* x, const float* a, int a_splits, const float* b, i
 }
 
 int kvcm_head_norm_gate(const float* o, int ldo, const float* g, int ldg, const float* w, void* out, int out_dtype,
-                        int ldout, int T, int heads, int d, float eps, hipStream_t s) {
+                        int ldout, int T, int heads, int d, float eps, int gate_silu, hipStream_t s) {
   if (T == 0) return 0;
   KVCM_REQUIRE(T > 0 && heads > 0 && d > 0, "head_norm_gate: bad sizes T=%d heads=%d d=%d", T, heads, d);
   KVCM_REQUIRE(ldo >= heads * d && ldg >= heads * d && ldout >= heads * d, "head_norm_gate: row strides too small");
@@ -271,10 +272,10 @@ int kvcm_head_norm_gate(const float* o, int ldo, const float* g, int ldg, const 
   KVCM_REQUIRE(blocks < (1ll << 31), "head_norm_gate: too many rows");
   if (out_dtype == kF32)
     head_norm_gate_kernel<float><<<static_cast<unsigned>(blocks), 256, 0, s>>>(o, ldo, g, ldg, w, static_cast<float*>(out),
-                                                                                ldout, items, heads, d, eps);
+                                                                                ldout, items, heads, d, eps, gate_silu);
   else if (out_dtype == kBF16)
     head_norm_gate_kernel<bf16_t><<<static_cast<unsigned>(blocks), 256, 0, s>>>(o, ldo, g, ldg, w, static_cast<bf16_t*>(out),
-                                                                                 ldout, items, heads, d, eps);
+                                                                                 ldout, items, heads, d, eps, gate_silu);
   else KVCM_REQUIRE(false, "head_norm_gate: unknown output dtype %d", out_dtype);
   return launch_status("head_norm_gate");
 }

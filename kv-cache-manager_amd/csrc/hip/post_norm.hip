@@ -5,8 +5,9 @@
 //                    dtype for the sublayer that reads them next, one launch for all of it.  y may be the un-added
 //                    slices of a product that was split along K: they are added here, in their order.  With a row
 //                    gather (the model's last norm, on the rows whose logits are wanted) nothing is written back.
-//   head_norm_store  what an attention with a norm per head does between its projection and its pages: biases, each q and
-//                    k head divided by its own root mean square and multiplied by one weight of the head's size, the query
+//   head_norm_store  what an attention with a norm per head does between its projection and its pages: biases, a rotation by
+//                    position of a part of each q and k head, each q and k head divided by its own root mean square and
+//                    multiplied by one weight of the head's size (or by none), the query
 //                    times a temperature that grows with the logarithm of its position, k to its page slot, and as values
 //                    either the projection's own or the keys as projected (before their norm).
 //
@@ -139,7 +140,8 @@ __global__ void __launch_bounds__(kPostThreads)
 template <class T>
 __global__ void __launch_bounds__(256)
     head_norm_store_kernel(const float* __restrict__ src, int ld, const float* __restrict__ bias, const float* __restrict__ wq,
-                           const float* __restrict__ wk, float eps, const int* __restrict__ positions, float temp_coef,
+                           const float* __restrict__ wk, float eps, int plain_norm, const float2* __restrict__ cos_sin, int rot, int halves,
+                           const int* __restrict__ positions, float temp_coef,
                            int temp_every, int values_are_keys, const int* __restrict__ slots, T* __restrict__ q_out, int ldq,
                            T* __restrict__ kcache, T* __restrict__ vcache, long long items, int nh, int nkv, int d, int dv, int B) {
   const long long item = static_cast<long long>(blockIdx.x) * (256 / kWave) + threadIdx.x / kWave;
@@ -160,11 +162,22 @@ __global__ void __launch_bounds__(256)
   if (!query && slot < 0) return;
   const int at = part * d;
   const float* w = query ? wq : wk;
+  const float2* cs = cos_sin + size_t(row) * (rot / 2);
+  auto projected = [&](int i) { return r[at + i] + (bias ? bias[at + i] : 0.f); };
+  auto entry = [&](int i) {      // the head's entry after the rotation
+    const float x = projected(i);
+    if (i >= rot) return x;      // (rot is even: the partner lies inside the rotated part too)
+    const int hr = rot / 2;
+    const bool second = halves ? i >= hr : (i & 1);
+    const float y = projected(halves ? (second ? i - hr : i + hr) : (i ^ 1));
+    const float2 a = cs[halves ? (second ? i - hr : i) : i / 2];
+    return second ? __fmaf_rn(x, a.x, __fmul_rn(y, a.y)) : __fmaf_rn(x, a.x, -__fmul_rn(y, a.y));
+  };
   float inv = 1.f;
-  if (w) {
+  if (w || plain_norm) {
     float ss = 0.f;
     for (int i = lane; i < d; i += kWave) {
-      const float x = r[at + i] + (bias ? bias[at + i] : 0.f);
+      const float x = entry(i);
       ss = fmaf(x, x, ss);
     }
     inv = 1.0f / sqrtf(wave_sum(ss) / float(d) + eps);
@@ -173,16 +186,16 @@ __global__ void __launch_bounds__(256)
     float temp = 1.f;
     if (temp_every > 0) temp = fmaf(temp_coef, logf(float((positions[row] + 1) / temp_every + 1)), 1.0f);
     for (int i = lane; i < d; i += kWave) {
-      const float x = r[at + i] + (bias ? bias[at + i] : 0.f);
-      store_f(q_out + size_t(row) * ldq + at + i, (w ? x * inv * w[i] : x) * temp);
+      const float x = entry(i) * inv;
+      store_f(q_out + size_t(row) * ldq + at + i, (w ? x * w[i] : x) * temp);
     }
     return;
   }
   const int head = part - nh;
   for (int i = lane; i < d; i += kWave) {
-    const float x = r[at + i] + (bias ? bias[at + i] : 0.f);
-    store_f(kcache + ((size_t(slot / B) * nkv + head) * B + slot % B) * d + i, w ? x * inv * w[i] : x);
-    if (values_are_keys) store_f(vcache + ((size_t(slot / B) * nkv + head) * dv + i) * B + slot % B, x);
+    const float x = entry(i) * inv;
+    store_f(kcache + ((size_t(slot / B) * nkv + head) * B + slot % B) * d + i, w ? x * w[i] : x);
+    if (values_are_keys) store_f(vcache + ((size_t(slot / B) * nkv + head) * dv + i) * B + slot % B, projected(i));
   }
 }
 
@@ -220,15 +233,18 @@ int kvcm_layernorm_post(float* x, const float* a, int a_splits, long long split_
 }
 
 // src [T, ld] 32-bit rows [q (nh*d) | k (nkv*d) | v (nkv*dv), the last only without values_are_keys]; bias: a row of the
-// same layout or null; wq, wk [d] or null (that kind of head passes un-normed); positions [T] (read with temp_every > 0:
+// same layout or null; wq, wk [d] or null (that kind of head passes un-normed, or with plain_norm is normed without a weight);
+// cos_sin [T, rot/2, 2] turns the first rot entries of every q and k head before the norm, by pairs (2i, 2i+1) or (halves)
+// (i, i + rot/2); positions [T] (read with temp_every > 0:
 // q <- q * (1 + temp_coef * ln(floor((p + 1) / temp_every) + 1))); slots [T] or null (nothing is stored).
 int kvcm_head_norm_store(const float* src, int ld, const float* bias, const float* wq, const float* wk, float eps,
-                         const int* positions, float temp_coef, int temp_every, int values_are_keys, const int* slots, void* q_out,
+                         int plain_norm, const float* cos_sin, int rot, int halves, const int* positions, float temp_coef, int temp_every, int values_are_keys, const int* slots, void* q_out,
                          int dtype, int ldq, void* kcache, void* vcache, int T, int nh, int nkv, int d, int dv, int B, hipStream_t s) {
   if (T == 0) return 0;
   KVCM_REQUIRE(T > 0 && nh > 0 && nkv > 0 && d > 0 && dv > 0 && B > 0 && src && q_out, "head_norm_store: bad sizes");
   KVCM_REQUIRE(!values_are_keys || dv == d, "head_norm_store: keys of %d entries cannot be values of %d", d, dv);
   KVCM_REQUIRE(ld >= (nh + nkv) * d + (values_are_keys ? 0 : nkv * dv) && ldq >= nh * d, "head_norm_store: row strides too small");
+  KVCM_REQUIRE(rot >= 0 && rot % 2 == 0 && rot <= d && (rot == 0 || cos_sin), "head_norm_store: %d rotated of %d entries is not supported", rot, d);
   KVCM_REQUIRE(temp_every <= 0 || positions, "head_norm_store: a temperature by position needs the positions");
   KVCM_REQUIRE(!slots || (kcache && vcache), "head_norm_store: slots without pages");
   const long long items = static_cast<long long>(T) * (nh + nkv + (values_are_keys ? 0 : nkv));
@@ -236,11 +252,11 @@ int kvcm_head_norm_store(const float* src, int ld, const float* bias, const floa
   KVCM_REQUIRE(blocks < (1ll << 31), "head_norm_store: too many rows");
   if (dtype == kF32)
     head_norm_store_kernel<float><<<static_cast<unsigned>(blocks), 256, 0, s>>>(
-        src, ld, bias, wq, wk, eps, positions, temp_coef, temp_every, values_are_keys, slots, static_cast<float*>(q_out), ldq,
+        src, ld, bias, wq, wk, eps, plain_norm, reinterpret_cast<const float2*>(cos_sin), rot, halves, positions, temp_coef, temp_every, values_are_keys, slots, static_cast<float*>(q_out), ldq,
         static_cast<float*>(kcache), static_cast<float*>(vcache), items, nh, nkv, d, dv, B);
   else if (dtype == kBF16)
     head_norm_store_kernel<bf16_t><<<static_cast<unsigned>(blocks), 256, 0, s>>>(
-        src, ld, bias, wq, wk, eps, positions, temp_coef, temp_every, values_are_keys, slots, static_cast<bf16_t*>(q_out), ldq,
+        src, ld, bias, wq, wk, eps, plain_norm, reinterpret_cast<const float2*>(cos_sin), rot, halves, positions, temp_coef, temp_every, values_are_keys, slots, static_cast<bf16_t*>(q_out), ldq,
         static_cast<bf16_t*>(kcache), static_cast<bf16_t*>(vcache), items, nh, nkv, d, dv, B);
   else KVCM_REQUIRE(false, "head_norm_store: unknown dtype %d", dtype);
   return launch_status("head_norm_store");

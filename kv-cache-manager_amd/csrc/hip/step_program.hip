@@ -124,10 +124,13 @@ const Entry kEntries[] = {
     KVCM_ENTRY(kvcm_head_norm_store),
     KVCM_ENTRY(kvcm_gemm_heads),
     KVCM_ENTRY(kvcm_act_rows),
+    KVCM_ENTRY(kvcm_stream_terms),
+    KVCM_ENTRY(kvcm_group_norm_gate),
+    KVCM_ENTRY(kvcm_gated_state),
 };
 #undef KVCM_ENTRY
 
-constexpr int kMaxArgs = 32;
+constexpr int kMaxArgs = 40;
 
 struct Launch {
   const Entry* entry;

@@ -119,6 +119,13 @@ int kvcm_core_keep_first(void* core, int g, int tokens) {
     return 0;
   });
 }
+// A windowed group whose queries see their own chunk of `size` tokens instead of a sliding window.
+int kvcm_core_chunk(void* core, int g, int size) {
+  return guarded([&] {
+    static_cast<Core*>(core)->kv->set_chunk(g, size);
+    return 0;
+  });
+}
 void kvcm_core_delete(void* c) { delete static_cast<Core*>(c); }
 
 int kvcm_core_policy_name(void* c, char* out, int cap) {

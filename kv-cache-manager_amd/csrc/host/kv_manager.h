@@ -29,6 +29,7 @@ struct GroupSpec {
   GroupKind kind = GroupKind::FullKV;
   int window = 0;      // WindowKV: a query at position p sees keys t with p - t < window
   int num_blocks = 0;  // pages in this group's pool (ignored for State)
+  int chunk = 0;       // WindowKV: > 0: a query at position p sees keys t of its own chunk only, t / chunk == p / chunk
   int keep_first = 0;  // WindowKV: queries also see the first keep_first tokens of their sequence, whatever the distance
 };
 
@@ -91,6 +92,13 @@ class KVManager {
     if (tokens > 0 && groups_[g].kind != GroupKind::WindowKV)
       throw std::invalid_argument("keep_first: only a windowed group gives pages back");
     groups_[g].keep_first = tokens;
+  }
+  // A windowed group whose queries see their own chunk of `size` tokens (counted from the sequence's start) instead of a
+  // window that slides: a chunk's pages are given back, all at once, when the next chunk begins.
+  void set_chunk(int g, int size) {
+    if (g < 0 || g >= num_groups() || size <= 0) throw std::invalid_argument("chunk: no such group, or a size that is not positive");
+    if (groups_[g].kind != GroupKind::WindowKV) throw std::invalid_argument("chunk: only a windowed group gives pages back");
+    groups_[g].chunk = size;
   }
 
   // Can every token now in seq.tokens be given room?
@@ -242,10 +250,12 @@ class PagedManager : public KVManager {
         seq.page_hashes.push_back(h);
       }
     }
-    // The next query sits at position >= num_computed and sees keys t > position - window.
+    // The next query sits at position >= num_computed and sees keys t > position - window, or its own chunk's.
     for (int g = 0; g < num_groups(); ++g) {
       if (groups_[g].kind != GroupKind::WindowKV) continue;
-      const int first_needed_token = std::max(0, seq.num_computed - groups_[g].window + 1);
+      const int chunk = groups_[g].chunk;
+      const int first_needed_token =
+          chunk > 0 ? seq.num_computed / chunk * chunk : std::max(0, seq.num_computed - groups_[g].window + 1);
       const int first_needed_page = std::min<int>(first_needed_token / bs_, static_cast<int>(seq.tables[g].size()));
       const int kept_pages = blocks_for(groups_[g].keep_first);      // pages that hold tokens every later query sees
       for (int b = std::max(seq.released_below[g], kept_pages); b < first_needed_page; ++b) {

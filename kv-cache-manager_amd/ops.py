@@ -90,9 +90,9 @@ def _declare(lib):
     fn("kvcm_gemm8", vp, i, vp, i, i, i, i, vp, i, f, vp, i, i, i, vp)
     fn("kvcm_gemm8_residual_norm", vp, i, vp, i, i, i, i, vp, vp, i, vp, vp, vp)
     fn("kvcm_embed_scaled", vp, vp, i, vp, i, i, i, f, vp)
-    fn("kvcm_gated_act", vp, i, vp, i, i, i, i, i, vp)
+    fn("kvcm_gated_act", vp, i, vp, vp, i, vp, i, i, i, i, i, vp)
     fn("kvcm_rmsnorm_chain", vp, vp, i, vp, i, C.c_longlong, vp, vp, f, vp, vp, vp, vp, i, i, i, f, vp)
-    fn("kvcm_head_norm_gate", vp, i, vp, i, vp, vp, i, i, i, i, i, f, vp)
+    fn("kvcm_head_norm_gate", vp, i, vp, i, vp, vp, i, i, i, i, i, f, i, vp)
     fn("kvcm_short_conv", vp, i, vp, vp, vp, vp, vp, i, i, vp, vp, vp, vp, vp, vp, i, i, i, i, i, vp)
     fn("kvcm_short_conv_state", vp, i, vp, vp, vp, vp, vp, vp, i, i, i, vp)
     fn("kvcm_rotary_pairs_table", vp, vp, i, i, f, vp)
@@ -106,11 +106,11 @@ def _declare(lib):
     fn("kvcm_head_gate", vp, i, i, vp, i, i, i, i, i, vp)
     fn("kvcm_rms_groups", vp, i, i, i, i, vp, f, vp, i, i, i, vp)
     fn("kvcm_layernorm_post", vp, vp, i, C.c_longlong, vp, f, vp, vp, vp, i, i, i, f, vp)
-    fn("kvcm_head_norm_store", vp, i, vp, vp, vp, f, vp, f, i, i, vp, vp, i, i, vp, vp, i, i, i, i, i, i, vp)
+    fn("kvcm_head_norm_store", vp, i, vp, vp, vp, f, i, vp, i, i, vp, f, i, i, vp, vp, i, i, vp, vp, i, i, i, i, i, i, vp)
     fn("kvcm_gemm_heads", vp, i, i, vp, vp, i, i, vp, i, i, i, i, i, vp)
     fn("kvcm_act_rows", vp, i, i, C.c_longlong, vp, i, i, i, i, i, vp)
     fn("kvcm_mlstm_scan", vp, i, vp, i, vp, i, vp, i, vp, i, vp, vp, f, f, vp, vp, vp, i, vp, vp, vp, vp, vp, vp, i, i, i, i, i, i, vp)
-    fn("kvcm_moe_route", vp, i, i, C.c_longlong, i, i, i, vp, vp, i, vp)
+    fn("kvcm_moe_route", vp, i, i, C.c_longlong, i, i, i, f, vp, vp, i, vp)
     fn("kvcm_moe_table_route", vp, vp, i, i, i, vp, vp, i, vp)
     fn("kvcm_moe_up", vp, i, i, vp, vp, vp, i, i, i, i, i, i, vp)
     fn("kvcm_moe_down", vp, i, vp, vp, vp, vp, vp, i, i, i, i, i, vp)
@@ -118,10 +118,15 @@ def _declare(lib):
     fn("kvcm_moe_grouped_max_tiles", i, i)
     fn("kvcm_moe_grouped", vp, i, vp, vp, vp, vp, vp, vp, vp, vp, vp, vp, i, i, i, i, i, i, i, vp)
     fn("kvcm_pool_update", vp, vp, i, vp, vp, vp, i, vp, vp, vp, i, i, i, i, i, i, i, vp)
-    fn("kvcm_attention_window_pool", vp, i, i, vp, i, vp, vp, vp, vp, vp, i, vp, vp, vp, vp, vp, i, i, i, i, i, i, i, f, i, i, i, i, f, vp)
+    fn("kvcm_attention_window_pool", vp, i, i, vp, i, vp, vp, vp, vp, vp, i, vp, vp, vp, vp, vp, i, i, i, i, i, i, i, f, i, i, i, i, f, i, i, f, vp)
     fn("kvcm_attention_window_pool_tiles_supported", i, i, i)
-    fn("kvcm_attention_window_pool_tiles", vp, i, vp, i, vp, vp, vp, vp, vp, i, vp, vp, vp, vp, vp, i, i, i, i, i, i, i, i, f, i, i, i, i, f, vp)
+    fn("kvcm_attention_window_pool_tiles", vp, i, vp, i, vp, vp, vp, vp, vp, i, vp, vp, vp, vp, vp, i, i, i, i, i, i, i, i, f, i, i, i, i, f, i, i, f, vp)
     fn("kvcm_selective_scan", vp, i, i, vp, i, vp, vp, i, i, i, vp, vp, vp, i, vp, i, vp, vp, vp, vp, i, i, i, i, i, i, vp, C.c_longlong, i, vp)
+    fn("kvcm_stream_terms", vp, vp, i, f, vp, i, f, vp, i, f, C.c_longlong, vp, vp, vp, vp, vp, i, i, i, f, vp)
+    fn("kvcm_group_norm_gate", vp, i, vp, i, vp, vp, i, i, i, i, i, f, vp)
+    fn("kvcm_gated_state", vp, i, vp, i, vp, i, vp, i, vp, i, vp, vp, vp, i, vp, i, vp, vp, vp, vp, i, i, i, i, i, i, i, i, vp, C.c_longlong, vp)
+    lib.kvcm_gated_state_carry_floats.restype = C.c_longlong
+    lib.kvcm_gated_state_carry_floats.argtypes = [i] * 7
     fn("kvcm_scan_prepare", vp, i, vp, vp, i, i, i, vp)
     fn("kvcm_delta_prepare", vp, i, vp, i, vp, vp, i, vp, i, vp, vp, vp, vp, i, i, i, vp)
     fn("kvcm_delta_scan", vp, i, vp, i, vp, i, vp, vp, vp, vp, i, vp, vp, vp, vp, i, i, i, i, vp)
@@ -987,14 +992,19 @@ def embed_scaled(ids, table, out, factor):
     _call("kvcm_embed_scaled", _ptr(ids), _ptr(table), _DT[table.dtype], _ptr(out), T, H, table.shape[0], float(factor), _stream())
 
 
-def gated_act(gate_up, out, activation):
-    """out[T, I] = act(gate) * up for 32-bit rows [gate (I) | up (I)]; act: "silu", "relu" or "gelu_tanh"."""
+def gated_act(gate_up, out, activation, bias=None, row_gate=None):
+    """out[T, I] = act(gate) * up for 32-bit rows [gate (I) | up (I)]; act: "silu", "relu" or "gelu_tanh".  ``bias`` (float32
+    [2I]): added to the rows first.  ``row_gate`` (float32 rows, column 0 is read): the result times sigmoid(row_gate[t, 0])."""
     T, I = out.shape
     _f32rows(gate_up, "gate_up", 2 * I)
     _rows2d(out, "out")
     _need(gate_up.shape[0] >= T and out.is_cuda, "gated_act: the rows do not agree")
     _need(activation in GATE_ACTIVATIONS, f"unknown activation {activation!r} ({sorted(GATE_ACTIVATIONS)})")
-    _call("kvcm_gated_act", _ptr(gate_up), gate_up.stride(0), _ptr(out), _DT[out.dtype], out.stride(0), T, I,
+    _f32(bias, "bias", 2 * I)
+    if row_gate is not None:
+        _f32rows(row_gate, "row_gate", 1)
+        _need(row_gate.shape[0] >= T, "gated_act: fewer gates than rows")
+    _call("kvcm_gated_act", _ptr(gate_up), gate_up.stride(0), _ptr(bias), _ptr(row_gate), row_gate.stride(0) if row_gate is not None else 0, _ptr(out), _DT[out.dtype], out.stride(0), T, I,
           GATE_ACTIVATIONS[activation], _stream())
 
 
@@ -1051,8 +1061,9 @@ def rmsnorm_chain(x, eps, pending=None, weight=None, out=None, rows=None, plain=
     return out
 
 
-def head_norm_gate(o, gate, weight, out, heads, d, eps):
-    """out[r, h, :] = n(o[r, h, :]) * weight[h, :] * sigmoid(gate[r, h, :])."""
+def head_norm_gate(o, gate, weight, out, heads, d, eps, activation="sigmoid"):
+    """out[r, h, :] = n(o[r, h, :]) * weight[h, :] * act(gate[r, h, :]), act: "sigmoid" or "silu"."""
+    _need(activation in ("sigmoid", "silu"), "head_norm_gate: the gate is 'sigmoid' or 'silu'")
     T = out.shape[0]
     _f32rows(o, "o", heads * d)
     _f32rows(gate, "gate", heads * d)
@@ -1060,7 +1071,7 @@ def head_norm_gate(o, gate, weight, out, heads, d, eps):
     _rows2d(out, "out")
     _need(o.shape[0] >= T and gate.shape[0] >= T and out.shape[1] >= heads * d and out.is_cuda, "head_norm_gate: shapes do not agree")
     _call("kvcm_head_norm_gate", _ptr(o), o.stride(0), _ptr(gate), gate.stride(0), _ptr(weight), _ptr(out), _DT[out.dtype],
-          out.stride(0), T, heads, d, float(eps), _stream())
+          out.stride(0), T, heads, d, float(eps), 1 if activation == "silu" else 0, _stream())
     return out
 
 
@@ -1207,12 +1218,15 @@ def pool_update(kcache, vcache, pk, pv, tables, table_stride, row_seq, positions
 
 
 def attention_window_pool(q, out, kcache, vcache, pk, pv, tables, table_stride, row_seq, ctx_lens, nh, nkv, d, dv, scale,
-                          window, P, head_scale=None, rows=None, keep_first=0, softcap=0.0, dist_slope=None, gate=None):
+                          window, P, head_scale=None, rows=None, keep_first=0, softcap=0.0, dist_slope=None, gate=None, chunk=0, sink=False,
+                          out_scale=1.0):
     """out[r, h] = softmax over the last ``window`` tokens, the sequence's first ``keep_first`` tokens and the pooled
     blocks of P tokens before the window (window 0: every token, no blocks) of (q . k) * scale * head_scale[h], times the
     values.  ``softcap`` c > 0: the scores are capped first, c tanh(score / c).  ``dist_slope`` (float32 [nh]): a bias that
     grows with the distance is taken off the scores, slope[h] * (query position - key position).  ``gate`` (float32 rows of
-    >= nh*dv): the output is multiplied element by element with sigmoid(gate) before it is stored."""
+    >= nh*dv): the output is multiplied element by element with sigmoid(gate) before it is stored.  ``chunk`` > 0 (window 0):
+    a row at position i sees the tokens j <= i with j // chunk == i // chunk.  ``sink``: one is added to the softmax's
+    denominator (a key of score 0 without a value).  ``out_scale``: a factor on the output."""
     _dev(q, out, kcache, vcache, tables, row_seq, ctx_lens)
     _rows2d(q, "q")
     _rows2d(out, "out")
@@ -1231,7 +1245,7 @@ def attention_window_pool(q, out, kcache, vcache, pk, pv, tables, table_stride, 
     _call("kvcm_attention_window_pool", _ptr(q), _DT[q.dtype], q.stride(0), _ptr(out), out.stride(0), _ptr(kcache), _ptr(vcache),
           _ptr(pk), _ptr(pv), _ptr(tables), table_stride, _ptr(row_seq), _ptr(ctx_lens), _ptr(head_scale), _ptr(dist_slope), _ptr(gate),
           gate.stride(0) if gate is not None else 0, T, nh, nkv, d, dv,
-          B, float(scale), int(window), int(P), E, int(keep_first), float(softcap or 0.0), _stream())
+          B, float(scale), int(window), int(P), E, int(keep_first), float(softcap or 0.0), int(chunk), 1 if sink else 0, float(out_scale), _stream())
 
 
 def attention_window_pool_tiles_supported(d, dv, dtype, block_size):
@@ -1240,7 +1254,8 @@ def attention_window_pool_tiles_supported(d, dv, dtype, block_size):
 
 
 def attention_window_pool_tiles(q, out, kcache, vcache, pk, pv, tables, table_stride, run_start, seq_start, num_seqs, max_run,
-                                nh, nkv, d, dv, scale, window, P, head_scale=None, keep_first=0, softcap=0.0, dist_slope=None, gate=None):
+                                nh, nkv, d, dv, scale, window, P, head_scale=None, keep_first=0, softcap=0.0, dist_slope=None, gate=None,
+                                chunk=0, sink=False, out_scale=1.0):
     """``attention_window_pool`` for steps whose sequences run several consecutive positions: 64 rows of a run and one
     head per workgroup on the matrix cores (bfloat16 only).  Every row of every run is computed, single rows too."""
     _dev(q, out, kcache, vcache, tables, run_start, seq_start)
@@ -1260,7 +1275,7 @@ def attention_window_pool_tiles(q, out, kcache, vcache, pk, pv, tables, table_st
     _call("kvcm_attention_window_pool_tiles", _ptr(q), q.stride(0), _ptr(out), out.stride(0), _ptr(kcache), _ptr(vcache), _ptr(pk),
           _ptr(pv), _ptr(tables), table_stride, _ptr(run_start), _ptr(seq_start), _ptr(head_scale), _ptr(dist_slope), _ptr(gate),
           gate.stride(0) if gate is not None else 0, num_seqs, max_run, nh, nkv,
-          d, dv, B, float(scale), int(window), int(P), E, int(keep_first), float(softcap or 0.0), _stream())
+          d, dv, B, float(scale), int(window), int(P), E, int(keep_first), float(softcap or 0.0), int(chunk), 1 if sink else 0, float(out_scale), _stream())
 
 
 SCAN_PIECE = 128      # rows of a piece when long runs are walked in pieces
@@ -1496,12 +1511,16 @@ def layernorm_post(x, weight, eps, alpha=1.0, add=None, out=None, rows=None):
 
 
 def head_norm_store(qkv, q_out, nh, nkv, d, dv, eps, q_weight=None, k_weight=None, bias=None, positions=None, temp_coef=0.0,
-                    temp_every=0, values_are_keys=False, slots=None, kcache=None, vcache=None, rows=None):
+                    temp_every=0, values_are_keys=False, slots=None, kcache=None, vcache=None, rows=None, plain_norm=False, cos_sin=None,
+                    rot=0, halves=False):
     """qkv: 32-bit rows [q (nh*d) | k (nkv*d) | v (nkv*dv)] (no v with ``values_are_keys``); ``bias``: a float32 row of
     that layout, added first.  Every q and k head is divided by its own root mean square (eps inside the root) and
     multiplied by ``q_weight`` / ``k_weight`` [d] (None: that kind passes); with ``temp_every`` > 0 the query is then
     multiplied by 1 + temp_coef * ln(floor((position + 1) / temp_every) + 1).  q goes to q_out [T, nh*d], k to its page
-    slot, and as values the projection's own or, with ``values_are_keys``, the keys as projected, before their norm."""
+    slot, and as values the projection's own or, with ``values_are_keys``, the keys as projected, before their norm.
+    ``plain_norm``: heads without a weight are normed too, not passed.  ``rot`` > 0: before the norm the first ``rot`` entries
+    of every q and k head are turned with the table ``cos_sin`` [T, rot/2, 2], by interleaved pairs or (``halves``) by pairs
+    (i, i + rot/2)."""
     T = q_out.shape[0] if rows is None else rows
     width = (nh + nkv) * d + (0 if values_are_keys else nkv * dv)
     _f32rows(qkv, "qkv", width)
@@ -1522,7 +1541,11 @@ def head_norm_store(qkv, q_out, nh, nkv, d, dv, eps, q_weight=None, k_weight=Non
         B = kcache.shape[2]
         _need(vcache is not None and vcache.dtype == q_out.dtype and vcache.is_contiguous()
               and tuple(vcache.shape) == (kcache.shape[0], nkv, dv, B), "value cache must be [pages, nkv, dv, block_size]")
-    _call("kvcm_head_norm_store", _ptr(qkv), qkv.stride(0), _ptr(bias), _ptr(q_weight), _ptr(k_weight), float(eps), _ptr(positions),
+    if rot:
+        _need(cos_sin is not None and cos_sin.dtype == torch.float32 and cos_sin.is_contiguous() and cos_sin.is_cuda
+              and cos_sin.numel() >= T * rot, "cos_sin must be float32 [rows, rot/2, 2]")
+    _call("kvcm_head_norm_store", _ptr(qkv), qkv.stride(0), _ptr(bias), _ptr(q_weight), _ptr(k_weight), float(eps),
+          1 if plain_norm else 0, _ptr(cos_sin) if rot else 0, int(rot), 1 if halves else 0, _ptr(positions),
           float(temp_coef), int(temp_every), 1 if values_are_keys else 0, _ptr(slots), _ptr(q_out), _DT[q_out.dtype], q_out.stride(0),
           _ptr(kcache), _ptr(vcache), T, nh, nkv, d, dv, B, _stream())
 
@@ -1590,11 +1613,11 @@ def mlstm_scan(q, k, v, gate_in, gate_keep, in_bias, keep_bias, cap, q_scale, co
     return o
 
 
-def moe_route(logits, experts, top, chosen, weight, rows=None, over_chosen=False):
+def moe_route(logits, experts, top, chosen, weight, rows=None, over_chosen=False, factor=1.0):
     """chosen[T, top] (int32) and weight[T, top] (float32): the ``top`` experts with the largest softmax scores over all
     ``experts`` of each row's 32-bit router logits, best first, with those scores; ``over_chosen``: with the softmax over
     the chosen logits alone instead (the weights of a row add up to one).  ``logits`` may be PartialSums (a router product
-    that was split along K): the slices are added as they are read."""
+    that was split along K): the slices are added as they are read.  ``factor``: a constant on the weights."""
     T = chosen.shape[0] if rows is None else rows
     splits, stride = 1, 0
     if isinstance(logits, PartialSums):
@@ -1609,7 +1632,7 @@ def moe_route(logits, experts, top, chosen, weight, rows=None, over_chosen=False
           "chosen must be int32 [T, top]")
     _need(weight.dtype == torch.float32 and weight.is_contiguous() and weight.is_cuda and tuple(weight.shape) == tuple(chosen.shape),
           "weight must be float32 [T, top]")
-    _call("kvcm_moe_route", _ptr(logits), ld, splits, stride, experts, top, 1 if over_chosen else 0, _ptr(chosen), _ptr(weight),
+    _call("kvcm_moe_route", _ptr(logits), ld, splits, stride, experts, top, 1 if over_chosen else 0, float(factor), _ptr(chosen), _ptr(weight),
           T, _stream())
 
 
@@ -1689,3 +1712,117 @@ def moe_grouped(h, w_up, w_down, chosen, weight, order, tiles, act, y, out, gate
     _call("kvcm_moe_grouped", _ptr(h), h.stride(0), _ptr(w_up), _ptr(w_down), _ptr(chosen), _ptr(weight), _ptr(order), _ptr(tiles),
           _ptr(act), _ptr(y), _ptr(add), _ptr(out), T, K, F, H, top, E, 1 if gated else 0, _stream())
     return out
+
+
+# --------------------------------- a stream whose layers' sublayers all read one normed copy of it; gated states
+class StreamTerms:
+    """Sublayer outputs that are still to be added to the residual stream: ``terms`` is a list of (value, factor), a value
+    being a float32 tensor [T, H] or the un-added slices of a split product (PartialSums), and ``bias`` a float32 row [H] or
+    None.  ``stream_terms`` adds them in the launch that norms the stream for its next reader (up to three terms)."""
+
+    MOST = 3
+
+    def __init__(self, terms=(), bias=None):
+        self.terms, self.bias = list(terms), bias
+
+    @classmethod
+    def of(cls, value):
+        """A part's result (None, a tensor, PartialSums, or StreamTerms) as StreamTerms."""
+        if value is None:
+            return cls()
+        if isinstance(value, cls):
+            return value
+        if isinstance(value, BiasedOutput):
+            return cls([(value.value, 1.0)], value.bias)
+        return cls([(value, 1.0)])
+
+    def plus(self, other):
+        other = StreamTerms.of(other)
+        _need(self.bias is None or other.bias is None, "StreamTerms: one constant row at most")
+        return StreamTerms(self.terms + other.terms, self.bias if other.bias is None else other.bias)
+
+
+def stream_terms(x, eps, add=None, again=None, weight=None, out=None, rows=None):
+    """x <- x + sum of the terms (StreamTerms or None), then + ``again`` (float32 [T, H] or None), written back unless ``rows``
+    gathers; out[r] = x[src] / sqrt(mean(x[src]^2) + eps) * weight, src = rows[r] or r.  All 32-bit, ``out`` rounded once."""
+    _need(x.dtype == torch.float32 and x.is_contiguous() and x.is_cuda and x.dim() == 2, "x must be contiguous float32 [T, H]")
+    T, H = x.shape
+    add = StreamTerms() if add is None else add
+    _need(len(add.terms) <= StreamTerms.MOST, f"stream_terms: {len(add.terms)} terms are not supported (up to {StreamTerms.MOST})")
+    flat = []
+    for value, factor in add.terms:
+        splits = 1
+        if isinstance(value, PartialSums):
+            _need(value.rows == T and value.cols == H, "a term's partial sums must match x")
+            value, splits = value.data, value.splits
+            _f32(value, "a term's partial sums", splits * T * H)
+        else:
+            _need(value.dtype == torch.float32 and value.is_contiguous() and value.is_cuda and tuple(value.shape) == (T, H), "a term must be float32 like x")
+        flat += [_ptr(value), splits, float(factor)]
+    flat += [0, 1, 0.0] * (StreamTerms.MOST - len(add.terms))
+    _f32(add.bias, "the constant row", H)
+    if again is not None:
+        _need(again.dtype == torch.float32 and again.is_contiguous() and again.is_cuda and tuple(again.shape) == (T, H), "again must be float32 like x")
+    R = T
+    if out is not None:
+        _need(out.is_cuda and out.is_contiguous() and out.dim() == 2 and out.shape[1] == H, "out must be contiguous [R, H]")
+        _need(weight is not None, "stream_terms: a normed output needs its weight")
+        _f32(weight, "the norm weight", H)
+        R = out.shape[0]
+        if rows is not None:
+            _i32(rows, "rows", R)
+        else:
+            _need(R == T, "stream_terms: the output must have the stream's rows")
+    else:
+        _need(rows is None, "stream_terms: gathered rows need an output")
+    _call("kvcm_stream_terms", _ptr(x), *flat, T * H, _ptr(add.bias), _ptr(again), _ptr(rows), _ptr(weight), _ptr(out),
+          _DT[out.dtype] if out is not None else 0, R, H, float(eps), _stream())
+    return out
+
+
+def group_norm_gate(y, z, weight, out, groups, size, eps):
+    """out[t, g*size + i] = n(y * silu(z))[i of group g] * weight, n: division by the group's own root mean square; y, z
+    float32 rows of groups*size, out rows of any stored dtype."""
+    T = out.shape[0]
+    _f32rows(y, "y", groups * size)
+    _f32rows(z, "z", groups * size)
+    _f32(weight, "weight", groups * size)
+    _rows2d(out, "out")
+    _need(y.shape[0] >= T and z.shape[0] >= T and out.shape[1] >= groups * size and out.is_cuda, "group_norm_gate: shapes do not agree")
+    _call("kvcm_group_norm_gate", _ptr(y), y.stride(0), _ptr(z), z.stride(0), _ptr(weight), _ptr(out), _DT[out.dtype], out.stride(0), T,
+          groups, size, float(eps), _stream())
+    return out
+
+
+GATED_STATE_PIECE = 128      # rows of a piece when long runs are walked in pieces
+
+
+def gated_state_carry_floats(rows, seqs, heads, dk, dv, delta, piece=GATED_STATE_PIECE):
+    """32-bit values of scratch that ``gated_state`` needs to walk a step of this shape in pieces."""
+    return int(lib().kvcm_gated_state_carry_floats(rows, seqs, heads, dk, dv, 1 if delta else 0, piece))
+
+
+def gated_state(q, k, v, a, dt_bias, a_log, o, state, step, heads, groups, dk, dv, b=None, d_skip=None, carry=None, piece=None):
+    """A matrix state per head with one decay per head and token over the step's runs (csrc/hip/gated_state.hip).  q, k
+    [T, groups*dk], v [T, heads*dv], a [T, heads]: float32 rows; state [slots, heads, dk, dv].  With ``b`` (float32 rows
+    [T, heads]): the gated delta rule, q and k made unit vectors (q times dk^-1/2), g = exp(-exp(a_log) softplus(a + dt_bias)),
+    S <- g S, S += k (sigmoid(b) (v - S^T k))^T, o = S^T q.  With ``d_skip`` [heads]: dt = softplus(a + dt_bias),
+    S <- exp(-exp(a_log) dt) S + dt k v^T, o = S^T q + d_skip v.  ``carry`` (float32 scratch of ``gated_state_carry_floats``):
+    runs are walked in pieces of ``piece`` rows, all pieces at once."""
+    T = o.shape[0]
+    delta = b is not None
+    _need(delta != (d_skip is not None), "gated_state: give b (the delta rule) or d_skip (the state-space recurrence)")
+    for t, n, c in ((q, "q", groups * dk), (k, "k", groups * dk), (v, "v", heads * dv), (a, "a", heads), (o, "o", heads * dv)) + (((b, "b", heads),) if delta else ()):
+        _f32rows(t, n, c)
+        _need(t.shape[0] >= T, f"{n} has too few rows")
+    for t, n in ((dt_bias, "dt_bias"), (a_log, "a_log"), (d_skip, "d_skip")):
+        _f32(t, n, heads)
+    _need(state.dtype == torch.float32 and state.is_contiguous() and state.is_cuda and tuple(state.shape[1:]) == (heads, dk, dv),
+          "state must be float32 [slots, heads, dk, dv]")
+    piece = (GATED_STATE_PIECE if piece is None else int(piece)) if carry is not None else 0
+    _f32(carry, "carry")
+    _call("kvcm_gated_state", _ptr(q), q.stride(0), _ptr(k), k.stride(0), _ptr(v), v.stride(0), _ptr(a), a.stride(0), _ptr(b),
+          b.stride(0) if delta else 0, _ptr(dt_bias), _ptr(a_log), _ptr(d_skip), 1 if delta else 0, _ptr(o), o.stride(0), _ptr(state),
+          _ptr(step.run_start), _ptr(step.seq_start), _ptr(step.state_slots), step.seqs, heads, groups, dk, dv, T, piece,
+          int(step.max_run), _ptr(carry), carry.numel() if carry is not None else 0, _stream())
+    return o

@@ -83,13 +83,19 @@ class KVCacheNeed:
     of a value where it differs from a key's (0: the same).  ``pool`` > 0: beside the tokens, every page keeps
     one 32-bit mean key and mean value for each block of ``pool`` tokens whose last token it holds
     (ceil(block_size / pool) entries a page), for attentions that see far blocks as one key.  ``keep_first`` > 0
-    (with a window): every query also sees the first ``keep_first`` tokens of its sequence, so their pages stay."""
+    (with a window): every query also sees the first ``keep_first`` tokens of its sequence, so their pages stay.
+    ``chunk`` > 0 (without a window): a query at position p sees the keys at t <= p of its own chunk, t // chunk == p // chunk."""
     num_kv_heads: int
     head_dim: int
     window: int = 0
     value_dim: int = 0
     pool: int = 0
     keep_first: int = 0
+    chunk: int = 0
+
+    def __post_init__(self):
+        if self.chunk and (self.window or self.pool or self.keep_first):
+            raise ValueError("a chunked cache has no window, no pooled blocks and keeps no first tokens")
 
 
 @dataclass(frozen=True)
@@ -107,6 +113,15 @@ class BuildContext:
     hidden_size: int
     block_size: int
     ops: object                 # the kernel module (kvcm_amd.ops)
+    derived: dict = field(default_factory=dict)      # tensors that parts make of their weights, by who made them
+
+    def derive(self, part, name, make):
+        """``make()``'s tensor, made once for all parts of one kind, prefix and parameters: parts of layers that run again share
+        not only the checkpoint's tensors but what is made of them (fused, padded, interleaved) as well."""
+        key = (type(part).__name__, part.prefix, repr(sorted(part.params.items(), key=lambda kv: kv[0])), name)
+        if key not in self.derived:
+            self.derived[key] = make()
+        return self.derived[key]
 
 
 # ------------------------------------------------------------------------------------- step
@@ -307,6 +322,29 @@ class FeedForward(Part):
     accepts_normed_rows = False      # as Mixer.accepts_normed_rows
 
     def forward(self, step, h):
+        raise NotImplementedError
+
+
+class JoinableEnds:
+    """A sublayer (a Mixer or a FeedForward) whose first operation is a product of its input rows h and whose last is a product
+    too, and which can leave both to whoever drives it: several sublayers of the same h then share one product at each end
+    (parts/joined_parts.py).  Built with the param ``joined`` it declares neither matrix itself."""
+
+    def in_sources(self):
+        """((checkpoint name, (rows, H)), ...): what h is multiplied with, in the order of the columns ``between`` gets."""
+        raise NotImplementedError
+
+    def out_source(self):
+        """(checkpoint name, (H, columns)): what the values that ``between`` leaves are multiplied with, or None."""
+        raise NotImplementedError
+
+    def out_bias(self):
+        """A float32 row [H] still to be added to the output, or None."""
+        return None
+
+    def between(self, step, h, proj, out):
+        """proj: 32-bit rows, h times the ``in_sources``; out: rows of the compute dtype (a view into wider rows) for the values
+        of the last product (None without one).  Returns a further 32-bit output [rows, H] to be added, or None."""
         raise NotImplementedError
 
 

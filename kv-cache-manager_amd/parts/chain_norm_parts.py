@@ -6,7 +6,7 @@ is one launch, an embedding with a factor, and a gated feed-forward with a choic
 import torch
 
 from ..registry import BLOCKS, EMBEDDINGS, FEED_FORWARDS, NORMS
-from .base import Block, Embedding, FeedForward, Norm, ParamSpec
+from .base import Block, Embedding, FeedForward, JoinableEnds, Norm, ParamSpec
 from .llama_parts import _linear
 
 
@@ -14,6 +14,14 @@ def f32_params(tensors):
     """Small tensors (norm weights, biases, per-head factors, convolution taps) as float32: widening what a
     checkpoint stores in 16 bits is exact, and the kernels that use them compute in 32-bit."""
     return {k: v.float().contiguous() for k, v in tensors.items()}
+
+
+def pad_rows(t, multiple=16):
+    """A matrix with zero rows appended up to a multiple (the few-row products take such widths)."""
+    extra = -t.shape[0] % multiple
+    if not extra:
+        return t
+    return torch.cat([t, torch.zeros(extra, t.shape[1], dtype=t.dtype, device=t.device)], 0)
 
 
 def linear32(ctx, step, x, w, name, keep_partial=False):
@@ -145,20 +153,45 @@ class ScaledTokenEmbedding(Embedding):
 
 
 @FEED_FORWARDS.register("gated_mlp")
-class GatedFeedForward(FeedForward):
+class GatedFeedForward(JoinableEnds, FeedForward):
     """down(act(gate(h)) * up(h)), gate and up as one fused projection whose 32-bit sums go straight into the
-    activation (steps of few rows in bfloat16 with silu: in the product's own epilogue).  params: intermediate_size, activation ("relu" | "silu" | "gelu_tanh"); gate, up, down: the
-    checkpoint names after the prefix (defaults "gate", "up", "down").  The result is 32-bit: a norm reads it."""
+    activation (steps of few rows in bfloat16 with silu and without biases: in the product's own epilogue).  params: intermediate_size, activation ("relu" | "silu" | "gelu_tanh"); gate, up, down: the
+    checkpoint names after the prefix (defaults "gate", "up", "down"); bias: all three projections have one (the tensor's
+    name + ".b").  The result is 32-bit: a norm reads it.  Offers its ends (JoinableEnds)."""
 
     capturable = True
 
-    def param_specs(self):
+    def in_sources(self):
         H, I, pre, p = self.ctx.hidden_size, self.params["intermediate_size"], self.prefix, self.params
-        return [ParamSpec("w_gate_up", ((pre + p.get("gate", "gate"), (I, H)), (pre + p.get("up", "up"), (I, H)))),
-                ParamSpec("w_down", ((pre + p.get("down", "down"), (H, I)),))]
+        return ((pre + p.get("gate", "gate"), (I, H)), (pre + p.get("up", "up"), (I, H)))
+
+    def out_source(self):
+        return (self.prefix + self.params.get("down", "down"), (self.ctx.hidden_size, self.params["intermediate_size"]))
+
+    def out_bias(self):
+        return self.w.get("b_down")
+
+    def param_specs(self):
+        specs = [] if self.params.get("joined") else [ParamSpec("w_gate_up", self.in_sources()), ParamSpec("w_down", (self.out_source(),))]
+        if self.params.get("bias"):
+            specs += [ParamSpec("b_gate_up", tuple((n + ".b", s[:1]) for n, s in self.in_sources()), role="bias"),
+                      ParamSpec("b_down", ((self.out_source()[0] + ".b", (self.ctx.hidden_size,)),), role="bias")]
+        return specs
+
+    def bind(self, tensors):
+        small = f32_params({k: v for k, v in tensors.items() if k.startswith("b_")})
+        super().bind({**tensors, **small})
+
+    def between(self, step, h, proj, out, row_gate=None):
+        """``row_gate`` (32-bit rows, column 0): the output times sigmoid of it, one gate per row."""
+        self.ctx.ops.gated_act(proj, out, self.params.get("activation", "silu"), bias=self.w.get("b_gate_up"), row_gate=row_gate)
 
     def forward(self, step, h):
         I, ops = self.params["intermediate_size"], self.ctx.ops
+        if self.params.get("bias"):
+            act = step.ws("gated_act", (step.rows, I))
+            self.between(step, h, linear32(self.ctx, step, h, self.w["w_gate_up"], "gated_gate_up"), act)
+            return ops.BiasedOutput(linear32(self.ctx, step, act, self.w["w_down"], "gated_out", keep_partial=True), self.w["b_down"])
         act = step.ws("gated_act", (step.rows, I))
         kind = self.params.get("activation", "silu")
         # few rows in bfloat16 with silu: the product that streams gate and up rows together and applies the activation

@@ -16,6 +16,7 @@ from ..registry import MIXERS, POSITIONS
 from . import paged_attention
 from .base import KVCacheNeed, Mixer, ParamSpec, PartSpec, PositionEncoding
 from .chain_norm_parts import f32_params, linear32
+from .chain_norm_parts import pad_rows as _pad_rows
 
 
 def rescaled_frequencies(dims, base, scaling=None):
@@ -107,14 +108,6 @@ class HalfSplitRotary(PositionEncoding):
 
     def apply(self, step, qkv, num_heads, num_kv_heads, head_dim, cache=None, slots=None):
         raise NotImplementedError("rotary_halves rotates inside ops.rotate_store (the mixer hands it pairs_table)")
-
-
-def _pad_rows(t, multiple=16):
-    """A matrix with zero rows appended up to a multiple (the few-row products take such widths)."""
-    extra = -t.shape[0] % multiple
-    if not extra:
-        return t
-    return torch.cat([t, torch.zeros(extra, t.shape[1], dtype=t.dtype, device=t.device)], 0)
 
 
 def _attend(mixer, step, q, attn, kc, vc, g, nh, nkv, d, dv, scale, window, keep_first=0, softcap=0.0, dist_slope=None, gate=None):

@@ -1,5 +1,6 @@
 """Mixers that carry a fixed-size 32-bit state per request instead of keys and values: the selective scan
-(with the short convolution in front of it) and the generalized delta rule.  Their states live in the
+(with the short convolution in front of it), the generalized delta rule, a matrix memory with exponential gates, the gated
+delta rule and the state-space recurrence with one decay per head (the last two behind a short convolution).  Their states live in the
 cache manager's state slots; a request's portion that starts at position 0 starts from zero.  Every size,
 constant and tensor name is a parameter.
 """
@@ -8,6 +9,7 @@ import torch
 from ..registry import MIXERS
 from .base import Mixer, ParamSpec, StateNeed
 from .chain_norm_parts import f32_params, linear32
+from .ends import EndsMixer
 from .llama_parts import _linear
 
 _SMALL = ("conv", "conv_bias", "dt_bias", "a_log", "d_skip", "a_bias", "w0", "w2", "norm")
@@ -187,3 +189,156 @@ class MatrixMemoryMixer(_StatefulMixer):
         gated = step.ws("memory_gated", (T, heads * dv))
         ops.head_norm_gate(o, g, w["norm"], gated, heads, dv, p["eps"])
         return linear32(self.ctx, step, gated, w["w_o"], "memory_out", keep_partial=True)      # the stream's next norm adds the slices
+
+
+class _ConvStateMixer(EndsMixer):
+    """A short convolution (silu) over some of the projected channels, then a matrix state per head with one decay per head
+    and token (ops.gated_state).  Keeps per request: the state and the convolution's last taps-1 inputs, both 32-bit."""
+
+    capturable = True
+
+    def state(self, name):
+        storage, index, _ = self.caches[name]
+        return storage.slots(index)
+
+    def needs(self, heads, dk, dv, taps, channels):
+        needs = {"state": StateNeed((heads, dk, dv), torch.float32)}
+        if taps > 1:
+            needs["conv"] = StateNeed((taps - 1, channels), torch.float32)
+        return needs
+
+    def convolved(self, step, x, bias=None):
+        """The convolution of the columns of x (as many as it has channels), 32-bit; its new inputs left in the slot."""
+        ops, weight = self.ctx.ops, self.w["conv"]
+        C, taps = weight.shape
+        mixed = step.ws(self.ends_name + "_conv", (step.rows, C), torch.float32)
+        state = self.state("conv") if taps > 1 else None
+        single = step.max_run == 1      # every sequence runs one row: the convolution leaves the new state itself
+        ops.short_conv(x, weight, mixed, step, state, bias_out=bias, activation="silu", update_state=single)
+        if not single:
+            ops.short_conv_state(x, state, step, taps)
+        return mixed
+
+    def carry(self, step, heads, dk, dv, delta):
+        """Scratch for walking long runs in pieces, sized for the engine's largest step; None for steps of short runs."""
+        ops = self.ctx.ops
+        if step.max_run < 4 * ops.GATED_STATE_PIECE:
+            return None
+        lim = step.limits
+        rows, seqs = max(step.rows, lim.max_tokens if lim else 0), max(step.seqs, lim.max_seqs if lim else 0)
+        return step.flat("gated_state_carry", ops.gated_state_carry_floats(rows, seqs, heads, dk, dv, delta))
+
+
+@MIXERS.register("gated_delta")
+class GatedDeltaMixer(_ConvStateMixer):
+    """The gated delta rule.  q, k (kv_heads heads of dim) and v (heads of vdim) pass a causal convolution per channel and
+    silu; q and k become unit vectors per head (x / sqrt(|x|^2 + 1e-6)), q times dim^(-1/2); head h reads q and k head
+    h / (heads / kv_heads).  beta = sigmoid(W_b h), g = exp(-exp(A_log) softplus(W_a h + dt_bias)), one each per head;
+    S <- g S, u = beta (v - S^T k), S <- S + k u^T, o = S^T q; every head's o is divided by its root mean square, times one
+    weight of the head's size that all heads share, times silu(W_g h), then the output projection.
+    params: heads, kv_heads, dim, vdim, conv (taps), eps, out_factor (on the output, default 1).
+    Tensors under the prefix: q, k, v (each + ".conv"), g, b, a, A_log, dt_bias, norm, o."""
+
+    ends_name = "gated_delta"
+
+    def __init__(self, params, prefix, ctx):
+        super().__init__(params, prefix, ctx)
+        p = params
+        self.nh, self.nkv, self.d, self.dv = p["heads"], p["kv_heads"], p["dim"], p["vdim"]
+        if self.nkv <= 0 or self.nh % self.nkv:
+            raise ValueError(f"gated_delta {prefix!r}: heads {self.nh} is not a multiple of kv_heads {self.nkv}")
+        self.qk = self.nkv * self.d
+        self.channels = 2 * self.qk + self.nh * self.dv
+
+    def in_sources(self):
+        H, pre, nv = self.ctx.hidden_size, self.prefix, self.nh * self.dv
+        return tuple((pre + n, (c, H)) for n, c in (("q", self.qk), ("k", self.qk), ("v", nv), ("g", nv), ("b", self.nh), ("a", self.nh)))
+
+    def out_source(self):
+        return (self.prefix + "o", (self.ctx.hidden_size, self.nh * self.dv))
+
+    def own_specs(self):
+        pre, K = self.prefix, self.params["conv"]
+        return [ParamSpec("conv", tuple((pre + n + ".conv", (c, K)) for n, c in (("q", self.qk), ("k", self.qk), ("v", self.nh * self.dv)))),
+                ParamSpec("a_log", ((pre + "A_log", (self.nh,)),), role="bias"),
+                ParamSpec("dt_bias", ((pre + "dt_bias", (self.nh,)),), role="bias"),
+                ParamSpec("norm", ((pre + "norm", (self.dv,)),), role="vector")]
+
+    def bind(self, tensors):
+        super().bind(tensors)
+        # the shared weight once per head, the output's factor in it
+        self.w["norm"] = (self.w["norm"].repeat(self.nh) * float(self.params.get("out_factor", 1.0))).contiguous()
+
+    def cache_needs(self):
+        return self.needs(self.nh, self.d, self.dv, self.params["conv"], self.channels)
+
+    def flops(self, rows, attended=0):
+        return super().flops(rows) + rows * self.nh * 7.0 * self.d * self.dv + 2.0 * rows * self.channels * self.params["conv"]
+
+    def between(self, step, h, proj, out):
+        ops, p, w = self.ctx.ops, self.params, self.w
+        nh, d, dv = self.nh, self.d, self.dv
+        mixed = self.convolved(step, proj)
+        q, k, v = mixed, mixed[:, self.qk:], mixed[:, 2 * self.qk:]
+        g, b, a = (proj[:, at:] for at in (self.channels, self.channels + nh * dv, self.channels + nh * dv + nh))
+        o = step.ws("gated_delta_o", (step.rows, nh * dv), torch.float32)
+        ops.gated_state(q, k, v, a, w["dt_bias"], w["a_log"], o, self.state("state"), step, nh, self.nkv, d, dv, b=b,
+                        carry=self.carry(step, nh, d, dv, True))
+        ops.head_norm_gate(o, g, w["norm"], out, nh, dv, p["eps"], activation="silu")
+
+
+@MIXERS.register("state_space_duality")
+class StateSpaceMixer(_ConvStateMixer):
+    """The state-space recurrence with one decay per head (Mamba-2's).  in -> [z | x | B | C | dt]; x, B and C pass a causal
+    convolution per channel (bias, silu); dt = softplus(dt + dt_bias); head h reads B and C of group h / (heads / groups);
+    S <- exp(-exp(A_log) dt) S + dt B x^T, y = S^T C + D x; y * silu(z), divided by the root mean square of each of
+    norm_groups equal parts, times a weight, then the output projection.
+    params: heads, vdim, state, groups, norm_groups, conv (taps), eps, out_factor (on the output, default 1).
+    Tensors under the prefix: in, conv, conv.b, A_log, dt_bias, D, norm, o."""
+
+    ends_name = "state_space"
+
+    def __init__(self, params, prefix, ctx):
+        super().__init__(params, prefix, ctx)
+        p = params
+        self.nh, self.dv, self.N, self.groups, self.norm_groups = p["heads"], p["vdim"], p["state"], p["groups"], p["norm_groups"]
+        self.inner = self.nh * self.dv
+        self.channels = self.inner + 2 * self.groups * self.N
+        if self.nh % self.groups or self.inner % self.norm_groups:
+            raise ValueError(f"state_space_duality {prefix!r}: {self.nh} heads in {self.groups} groups, {self.inner} channels in "
+                             f"{self.norm_groups} parts do not come out even")
+
+    def in_sources(self):
+        return ((self.prefix + "in", (self.inner + self.channels + self.nh, self.ctx.hidden_size)),)
+
+    def out_source(self):
+        return (self.prefix + "o", (self.ctx.hidden_size, self.inner))
+
+    def own_specs(self):
+        pre = self.prefix
+        return [ParamSpec("conv", ((pre + "conv", (self.channels, self.params["conv"])),)),
+                ParamSpec("conv_bias", ((pre + "conv.b", (self.channels,)),), role="bias"),
+                ParamSpec("a_log", ((pre + "A_log", (self.nh,)),), role="bias"),
+                ParamSpec("dt_bias", ((pre + "dt_bias", (self.nh,)),), role="bias"),
+                ParamSpec("d_skip", ((pre + "D", (self.nh,)),), role="vector"),
+                ParamSpec("norm", ((pre + "norm", (self.inner,)),), role="vector")]
+
+    def bind(self, tensors):
+        super().bind(tensors)
+        self.w["norm"] = (self.w["norm"] * float(self.params.get("out_factor", 1.0))).contiguous()
+
+    def cache_needs(self):
+        return self.needs(self.nh, self.N, self.dv, self.params["conv"], self.channels)
+
+    def flops(self, rows, attended=0):
+        return super().flops(rows) + rows * self.nh * 5.0 * self.N * self.dv + 2.0 * rows * self.channels * self.params["conv"]
+
+    def between(self, step, h, proj, out):
+        ops, p, w = self.ctx.ops, self.params, self.w
+        inner, GN = self.inner, self.groups * self.N
+        mixed = self.convolved(step, proj[:, inner:], bias=w["conv_bias"])
+        y = step.ws("state_space_y", (step.rows, inner), torch.float32)
+        ops.gated_state(mixed[:, inner + GN:], mixed[:, inner:], mixed, proj[:, inner + self.channels:], w["dt_bias"], w["a_log"], y,
+                        self.state("state"), step, self.nh, self.groups, self.N, self.dv, d_skip=w["d_skip"],
+                        carry=self.carry(step, self.nh, self.N, self.dv, False))
+        ops.group_norm_gate(y, proj, w["norm"], out, self.norm_groups, inner // self.norm_groups, p["eps"])

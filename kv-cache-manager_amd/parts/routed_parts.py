@@ -5,8 +5,8 @@ may run for every row beside them.  Every size, constant and tensor name is a pa
 import torch
 
 from ..registry import FEED_FORWARDS
-from .base import FeedForward, ParamSpec
-from .chain_norm_parts import linear32
+from .base import FeedForward, JoinableEnds, ParamSpec
+from .chain_norm_parts import linear32, pad_rows
 
 
 def interleave_gate_up(gate, up):
@@ -19,7 +19,7 @@ def interleave_gate_up(gate, up):
 
 
 @FEED_FORWARDS.register("routed_experts")
-class RoutedExperts(FeedForward):
+class RoutedExperts(JoinableEnds, FeedForward):
     """Which experts a row uses (``routing``):
       "softmax" (default)  router logits z = W_router h in 32-bit, scores s = softmax(z) over all experts; the ``top``
                            experts with the largest scores, weighted by their scores as they are (not renormalized)
@@ -29,7 +29,11 @@ class RoutedExperts(FeedForward):
       "relu2" (default)    W_down act(W_up h), act = the square of relu
       "silu_gated"         W_down (silu(W_gate h) * (W_up h))
     Experts have no biases.  ``shared``: a PartSpec of a feed-forward that runs for every row and is added (default none).
-    params: experts, top, ff, routing, activation, shared, vocab_size (rows of the table; default: as stored); router / table (the checkpoint name after the prefix, defaults
+    ``shared_gate``: the shared feed-forward's output is multiplied by sigmoid(W_sg h), one number per row (the tensor's name
+    after the prefix; default none).  ``route_factor``: a constant on the experts' weights (default 1).
+    Offers its ends (JoinableEnds): the router's product, the gate's and the shared feed-forward's first at one end, the shared
+    feed-forward's last at the other; the experts' sum is the further output.  With ``shared_gate`` it runs that way on its own too.
+    params: experts, top, ff, routing, activation, shared, shared_gate, route_factor, vocab_size (rows of the table; default: as stored); router / table (the checkpoint name after the prefix, defaults
     "router", "table"); expert (a pattern for an expert's prefix, default "e{}."), gate, up, down (names after it).
     The result is 32-bit."""
 
@@ -47,11 +51,34 @@ class RoutedExperts(FeedForward):
             raise ValueError(f"routed_experts {prefix!r}: activation {self.activation!r} is not supported (relu2 | silu_gated)")
         self.gated = self.activation == "silu_gated"
         sh = params.get("shared")
-        self.shared = FEED_FORWARDS.get(sh.kind)(sh.params, sh.prefix, ctx) if sh is not None else None
+        self.by_ends = bool(params.get("joined") or params.get("shared_gate"))
+        if self.by_ends and self.routing == "table":
+            raise ValueError(f"routed_experts {prefix!r}: a table's routing has no product to join")
+        if params.get("shared_gate") and sh is None:
+            raise ValueError(f"routed_experts {prefix!r}: a gate on a shared feed-forward needs one")
+        self.shared = None
+        if sh is not None:
+            self.shared = FEED_FORWARDS.get(sh.kind)({**sh.params, "joined": True} if self.by_ends else sh.params, sh.prefix, ctx)
+            if self.by_ends and not isinstance(self.shared, JoinableEnds):
+                raise ValueError(f"routed_experts {prefix!r}: the shared {sh.kind!r} does not offer its ends")
         self.F = params["ff"]
 
     def sub_parts(self):
         return (self.shared,) if self.shared is not None else ()
+
+    def in_sources(self):
+        H, p, pre = self.ctx.hidden_size, self.params, self.prefix
+        sources = self.shared.in_sources() if self.shared is not None else ()
+        sources += ((pre + p.get("router", "router"), (p["experts"], H)),)
+        if p.get("shared_gate"):
+            sources += ((pre + p["shared_gate"], (1, H)),)
+        return sources
+
+    def out_source(self):
+        return self.shared.out_source() if self.shared is not None else None
+
+    def out_bias(self):
+        return self.shared.out_bias() if self.shared is not None else None
 
     def param_specs(self):
         H, p, pre = self.ctx.hidden_size, self.params, self.prefix
@@ -63,8 +90,10 @@ class RoutedExperts(FeedForward):
             specs.append(ParamSpec("w_gate", tuple((n + p.get("gate", "gate"), (F, H)) for n in names)))
         if self.routing == "table":
             specs.append(ParamSpec("table", ((pre + p.get("table", "table"), (p.get("vocab_size", -1), p["top"])),), role="index", distinct_below=E))
-        else:
+        elif not self.by_ends:
             specs.append(ParamSpec("w_router", ((pre + p.get("router", "router"), (E, H)),)))
+        elif not p.get("joined"):
+            specs += [ParamSpec("w_in", self.in_sources()), ParamSpec("w_shared_out", (self.out_source(),))]
         return specs
 
     def bind(self, tensors):
@@ -72,14 +101,15 @@ class RoutedExperts(FeedForward):
         bound = {}
         if self.routing == "table":
             bound["table"] = tensors["table"].contiguous()
+        elif self.by_ends:
+            if "w_in" in tensors:
+                bound["w_in"] = self.ctx.derive(self, "w_in", lambda: pad_rows(tensors["w_in"]))
+                bound["w_shared_out"] = tensors["w_shared_out"]
         else:
-            r = tensors["w_router"]
-            extra = -r.shape[0] % 16      # the few-row products take widths that are multiples of 16; the route reads the first E
-            if extra:
-                r = torch.cat([r, torch.zeros(extra, r.shape[1], dtype=r.dtype, device=r.device)], 0)
-            bound["w_router"] = r
-        up, down = tensors["w_up"].view(E, F, H), tensors["w_down"].view(E, H, F)
-        if self.gated:
+            bound["w_router"] = pad_rows(tensors["w_router"])      # the route reads the first E
+
+        def gated_pair():
+            up, down = tensors["w_up"].view(E, F, H), tensors["w_down"].view(E, H, F)
             # gate and up as one matrix, rows interleaved sixteen at a time; columns that bring F to a multiple of 16 are zero
             # (silu(0) * 0 = 0, and the down matrix has zero columns there)
             gate, pad = tensors["w_gate"].view(E, F, H), -F % 16
@@ -87,9 +117,12 @@ class RoutedExperts(FeedForward):
                 zeros = torch.zeros(E, pad, H, dtype=up.dtype, device=up.device)
                 gate, up = torch.cat([gate, zeros], 1), torch.cat([up, zeros], 1)
                 down = torch.cat([down, torch.zeros(E, H, pad, dtype=down.dtype, device=down.device)], 2).contiguous()
-            up = interleave_gate_up(gate, up)
-            self.F = F + pad
-        bound["w_up"], bound["w_down"] = up, down
+            return interleave_gate_up(gate, up), down
+        if self.gated:
+            bound["w_up"], bound["w_down"] = self.ctx.derive(self, "gated_pair", gated_pair)
+            self.F = F + -F % 16
+        else:
+            bound["w_up"], bound["w_down"] = tensors["w_up"].view(E, F, H), tensors["w_down"].view(E, H, F)
         super().bind(bound)
 
     def bytes_read(self, rows):
@@ -97,15 +130,41 @@ class RoutedExperts(FeedForward):
         p, w = self.params, self.w
         reached = min(p["experts"], rows * p["top"])
         per_expert = (w["w_up"][0].numel() + w["w_down"][0].numel()) * w["w_up"].element_size()
-        routing = rows * p["top"] * 4 if self.routing == "table" else w["w_router"].numel() * w["w_router"].element_size()
+        if self.routing == "table":
+            routing = rows * p["top"] * 4
+        else:      # (joined, the router is counted where its product is)
+            routing = sum(w[n].numel() * w[n].element_size() for n in ("w_router", "w_in", "w_shared_out") if n in w)
         return routing + reached * per_expert
 
     def flops(self, rows, attended=0):
         p, H = self.params, self.ctx.hidden_size
-        router = 0 if self.routing == "table" else p["experts"] * H
+        router = 0 if self.routing == "table" or p.get("joined") else p["experts"] * H
+        if self.by_ends and not p.get("joined"):
+            router = self.w["w_in"].shape[0] * H + self.w["w_shared_out"].numel()
         return 2.0 * rows * (router + p["top"] * (3 if self.gated else 2) * p["ff"] * H)
 
+    def between(self, step, h, proj, out):
+        p = self.params
+        at = sum(shape[0] for _, shape in self.shared.in_sources()) if self.shared is not None else 0
+        if self.shared is not None:
+            if p.get("shared_gate"):
+                self.shared.between(step, h, proj, out, row_gate=proj[:, at + p["experts"]:])
+            else:
+                self.shared.between(step, h, proj, out)
+        return self._experts(step, h, proj[:, at:])
+
     def forward(self, step, h):
+        if self.by_ends:
+            proj = linear32(self.ctx, step, h, self.w["w_in"], "routed_in")
+            values = step.ws("routed_values", (step.rows, self.w["w_shared_out"].shape[1]))
+            experts = self.between(step, h, proj, values)
+            ops = self.ctx.ops
+            return ops.StreamTerms([(linear32(self.ctx, step, values, self.w["w_shared_out"], "routed_shared_out", keep_partial=True), 1.0),
+                                    (experts, 1.0)], self.out_bias())
+        return self._experts(step, h)
+
+    def _experts(self, step, h, logits=None):
+        """The experts' weighted sum, 32-bit [T, H]; ``logits``: the router's, where somebody else made them."""
         ops, p, w = self.ctx.ops, self.params, self.w
         E, top, F, T = p["experts"], p["top"], self.F, step.rows
         chosen = step.ws("routed_chosen", (T, top), torch.int32)
@@ -113,9 +172,11 @@ class RoutedExperts(FeedForward):
         if self.routing == "table":
             ops.moe_table_route(step.tokens, w["table"], top, chosen, weight, rows=T)
         else:
-            logits = linear32(self.ctx, step, h, w["w_router"], "routed_logits", keep_partial=True)      # the route adds the slices
-            ops.moe_route(logits, E, top, chosen, weight, rows=T, over_chosen=self.routing == "softmax_chosen")
-        add = self.shared.forward(step, h) if self.shared is not None else None      # 32-bit [T, H]: the experts' sum starts from it
+            if logits is None:
+                logits = linear32(self.ctx, step, h, w["w_router"], "routed_logits", keep_partial=True)      # the route adds the slices
+            ops.moe_route(logits, E, top, chosen, weight, rows=T, over_chosen=self.routing == "softmax_chosen",
+                          factor=p.get("route_factor", 1.0))
+        add = self.shared.forward(step, h) if self.shared is not None and not self.by_ends else None      # 32-bit [T, H]: the experts' sum starts from it
         H = self.ctx.hidden_size
         act = step.ws("routed_act", (T, top * F)).view(T * top, F)
         out = step.ws("routed_out", (T, H), torch.float32)
