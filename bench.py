@@ -3,7 +3,7 @@
   python bench.py [--gpus 1] [--steps K] [--warmup W] [--batch 8] [--prompt-len 512] [--layers L]
                   [--sizes tinyllama-1.1b|llama-2-7b|llama-3-8b] [--context-limit 2048] [--prefill-tokens 2048]
                   [--tune-products off|heuristic|all] [--no-points] [--only-prefill]
-  python bench.py --design kasuvik|furapel|fisesun|betirax [--design-sizes 2048,4096] [--layers 4] [--prefill-tokens 2048] [--steps K]
+  python bench.py --design kasuvik|furapel|fisesun|betirax|vugotar [--design-sizes 2048,4096] [--layers 4] [--prefill-tokens 2048] [--steps K]
 
 A "step" is one decode step of the whole engine (schedule, batch metadata, upload, model step on
 the GPU, sampling, download, update).  W untimed steps, then exactly K timed steps between two
@@ -27,6 +27,11 @@ matrix memory; gated experts named by a table per token id beside a shared exper
 per head, keys as values, a query temperature, a distance bias, a window and a gate per element; latent attention with a
 rotated key part and query latents; a dense feed-forward or gated experts weighted over the chosen logits beside a shared
 expert) beside the Fisesun and the Llama decoder.
+
+--design vugotar does the same for the Vugotar decoder (parallel layers of one norm: attention over chunks with a norm per head
+and a sink beside a gated delta rule, the state-space recurrence with one decay per head; a dense feed-forward with biases or
+gated experts weighted over the chosen ones beside a shared expert with a gate) beside the Kasuvik, the Betirax and the Llama
+decoder.
 """
 import argparse
 import json
@@ -255,6 +260,31 @@ def betirax_config(width, layers, vocab=32000):
                                     "norm": {"eps": 1e-6}, "postln_alpha": 2.0, "layers": listed})
 
 
+# Vugotar at a width: (value size of a delta head, state of the state-space layers, its groups, its norm parts, experts, experts a row)
+VUGOTAR_SIZES = {2048: (64, 64, 4, 4, 8, 2), 4096: (128, 128, 8, 8, 8, 2)}
+
+
+def vugotar_config(width, layers, vocab=32000):
+    """A Vugotar configuration at a width of DESIGN_SIZES: three layers of four have the two mixers side by side (chunks of the
+    other designs' window), the third of four is a state-space layer twice as wide inside as the model; the first and third of
+    four have a dense feed-forward, the others ``experts`` gated experts of which a row uses ``top`` and a shared expert (the
+    ``top`` experts a quarter each and the shared one half of the dense feed-forward's width)."""
+    from kvcm_amd.config.vugotar_config import VugotarConfig
+    nh, nkv, hd, ff, window = DESIGN_SIZES[width][:5]
+    vd, state, groups, norm_groups, experts, top = VUGOTAR_SIZES[width]
+    moe = {"kind": "moe", "expert": {"ff": ff // (2 * top)}, "router": {"experts": experts, "top": top, "scale": 1.5}, "shared": {"ff": ff // 2}}
+    dense = {"kind": "dense", "ff": ff}
+    left = {"heads": nh, "kv_heads": nkv, "dim": hd, "vdim": hd, "scale": hd ** -0.5, "mask": {"size": window}, "rot": {"dims": hd, "base": 500000.0}}
+    right = {"heads": nh, "kv_heads": nh // 2, "dim": hd, "vdim": vd, "conv": 4}
+    parallel = {"left": left, "right": right, "left_scale": 1.1, "right_scale": 0.6}
+    mamba2 = {"heads": 2 * width // hd, "vdim": hd, "state": state, "groups": groups, "norm_groups": norm_groups, "conv": 4}
+    listed = []
+    for i in range(layers):
+        mlp = dense if i % 2 == 0 else moe
+        listed.append({"type": "mamba2", "mixer": mamba2, "mlp": mlp} if i % 4 == 2 else {"type": "parallel", "mixer": parallel, "mlp": mlp})
+    return VugotarConfig.from_dict({"architecture": "Vugotar", "vocab": vocab, "width": width, "norm": {"eps": 1e-6}, "layers": listed})
+
+
 def design_main(args):
     import torch
     from kvcm_amd.config.engine_config import EngineConfig
@@ -269,7 +299,8 @@ def design_main(args):
     first = args.design
     record = {"metric": "prefill and decode tok/s of the %s decoder beside the %s at equal sizes"
                         % (first.capitalize(), {"kasuvik": "Llama decoder", "furapel": "Kasuvik and Llama decoders",
-                                                 "fisesun": "Furapel and Llama decoders", "betirax": "Fisesun and Llama decoders"}[first]), "dtype": key,
+                                                 "fisesun": "Furapel and Llama decoders", "betirax": "Fisesun and Llama decoders",
+                                                 "vugotar": "Kasuvik, Betirax and Llama decoders"}[first]), "dtype": key,
               "data": "synthetic", "layers": layers, "prefill_tokens": T, "prompt_len": args.prompt_len, "steps": steps, "sizes": {}}
     for width in [int(w) for w in args.design_sizes.split(",")]:
         if width not in DESIGN_SIZES:
@@ -283,10 +314,13 @@ def design_main(args):
             designs = {"fisesun": fisesun_config(width, layers), "furapel": furapel_config(width, layers), "llama": designs["llama"]}
         elif first == "betirax":
             designs = {"betirax": betirax_config(width, layers), "fisesun": fisesun_config(width, layers), "llama": designs["llama"]}
+        elif first == "vugotar":
+            designs = {"vugotar": vugotar_config(width, layers), "kasuvik": designs["kasuvik"], "betirax": betirax_config(width, layers),
+                       "llama": designs["llama"]}
         if args.design_alone:
             designs = {first: designs[first]}
         for name, cfg in designs.items():
-            arch = {"kasuvik": "Kasuvik", "furapel": "Furapel", "fisesun": "Fisesun", "betirax": "Betirax", "llama": "LlamaForCausalLM"}[name]
+            arch = {"kasuvik": "Kasuvik", "furapel": "Furapel", "fisesun": "Fisesun", "betirax": "Betirax", "vugotar": "Vugotar", "llama": "LlamaForCausalLM"}[name]
             tensors = random_tensors(arch, cfg, seed=0, dtype=dt, device="cuda:0")
             ec = EngineConfig(block_size=16, max_seq_len=limit, num_blocks=8 * limit // 16, max_num_seqs=8,
                               max_batched_tokens=max(4096, T + 64), dtype=args.dtype, max_logit_rows=64, beyond_max_position=True)
@@ -339,11 +373,12 @@ def main():
                     help="run nothing but the 2,048-token prefill (for a profiler); prints its record alone")
     ap.add_argument("--prefill-tokens", type=int, default=2048,
                     help="tokens of the prefill measurement (2,048 in the record; other lengths for sweeps)")
-    ap.add_argument("--design", default="llama", choices=["llama", "kasuvik", "furapel", "fisesun", "betirax"],
+    ap.add_argument("--design", default="llama", choices=["llama", "kasuvik", "furapel", "fisesun", "betirax", "vugotar"],
                     help="llama: the workload above (the default); kasuvik: prefill and decode of the Kasuvik decoder beside the "
                          "Llama decoder at equal sizes; furapel: the same for the Furapel decoder beside both; "
                          "fisesun: the same for the Fisesun decoder beside the Furapel and the Llama decoder; "
-                         "betirax: the same for the Betirax decoder beside the Fisesun and the Llama decoder "
+                         "betirax: the same for the Betirax decoder beside the Fisesun and the Llama decoder; "
+                         "vugotar: the same for the Vugotar decoder beside the Kasuvik, the Betirax and the Llama decoder "
                          "(--design-sizes, --layers, --prefill-tokens, --prompt-len, --steps)")
     ap.add_argument("--design-sizes", default="2048,4096", help="widths of the --design comparison (2048, 4096)")
     ap.add_argument("--design-alone", action="store_true", help="run the --design itself only, not the designs beside it (for a profiler)")
