@@ -10,7 +10,8 @@
 // here is 32-bit.  A run that starts at position 0 starts from zero without reading its slot.
 //
 // The walk takes one token after another.  A value column j of S needs S^T k of its own column only, so columns are spread
-// over lanes and workgroups (256 / G of them a workgroup, the key dimension of a column over G lanes); the tokens' vectors
+// over lanes and workgroups (JPT * 256 / G of them a workgroup, the key dimension of a column over G lanes, JPT columns a lane,
+// so that a staged q and k serve JPT columns; a column's operations do not depend on JPT); the tokens' vectors
 // are staged through LDS a few at a time, the next ones requested before the current are computed, and a token's scalars
 // (decay, rate, the lengths of its q and k) are made as its vectors are staged, so that no transcendental function and no
 // sum across the head sits in the chain from token to token.
@@ -45,15 +46,15 @@ struct StateArgs {
 __device__ __forceinline__ int piece_place(int run0, int s, int p, int piece) { return run0 / piece + s + p; }
 
 // ENDS: the first of the three launches (no outputs, a state of W columns from zero / identity, written to the carry)
-template <int DKP, int G, int TILE, bool DELTA, bool ENDS>
+template <int DKP, int G, int JPT, int TILE, bool DELTA, bool ENDS>
 __global__ void __launch_bounds__(256) gated_state_kernel(StateArgs A) {
-  constexpr int IPT = DKP / G, CB = 256 / G, V = 2 * DKP + CB, SC = 4;
+  constexpr int IPT = DKP / G, LC = 256 / G, CB = LC * JPT, KAT = ENDS ? 0 : DKP, V = KAT + DKP + CB, SC = 4;
   constexpr int PF = (TILE * V + 255) / 256;
-  __shared__ __attribute__((aligned(16))) float tile[TILE][V + SC];      // per token: q, k (zero beyond dk), v of these columns, scalars
+  __shared__ __attribute__((aligned(16))) float tile[TILE][V + SC];      // per token: q (not without outputs), k (zero beyond dk), v of these columns, scalars
   const int head = blockIdx.x / A.col_blocks, cb = blockIdx.x % A.col_blocks;
   const int s = blockIdx.y / A.pieces_per_seq, p = blockIdx.y % A.pieces_per_seq;
   const int dk = A.dk, dv = A.dv, W = ENDS && DELTA ? dv + dk : dv;
-  const int g = threadIdx.x % G, jl = threadIdx.x / G, j = cb * CB + jl;
+  const int g = threadIdx.x % G, jl = threadIdx.x / G, j0 = cb * CB + jl;      // this lane's columns: j0 + c * LC, c < JPT
   int r0 = A.run_start[s], r1 = A.run_start[s + 1];
   const int slot = A.state_slots[s];
   const int run0 = r0, run1 = r1;
@@ -65,26 +66,30 @@ __global__ void __launch_bounds__(256) gated_state_kernel(StateArgs A) {
   if (r1 <= r0) return;
   const bool last = r1 == run1;
   if (ENDS && (last || slot < 0)) return;      // nothing follows the last piece
-  const bool owns = j < W;
   if (slot < 0) {
-    if (owns && g == 0)
-      for (int row = r0; row < r1; ++row) A.o[size_t(row) * A.ldo + size_t(head) * dv + j] = 0.f;
+    if (g == 0)
+      for (int row = r0; row < r1; ++row)
+        for (int c = 0; c < JPT; ++c)
+          if (j0 + c * LC < dv) A.o[size_t(row) * A.ldo + size_t(head) * dv + j0 + c * LC] = 0.f;
     return;
   }
   const int group = head / (A.heads / A.groups);
   const bool fresh = A.seq_start[s] == 0;
-  float* st = A.state + ((size_t(slot) * A.heads + head) * dk) * dv + (owns ? j : 0);      // [i][j]
+  float* st = A.state + ((size_t(slot) * A.heads + head) * dk) * dv;                        // [i][j]
   const int CW = DELTA ? dv + dk : dv;                                                       // a carry's columns
   float* cst = nullptr;
-  if (pieces) cst = A.carry + ((size_t(piece_place(run0, s, p, A.piece)) * A.heads + head) * dk) * CW + (owns ? j : 0);
-  float S[IPT];
+  if (pieces) cst = A.carry + ((size_t(piece_place(run0, s, p, A.piece)) * A.heads + head) * dk) * CW;
+  float S[JPT][IPT];
 #pragma unroll
-  for (int il = 0; il < IPT; ++il) {
-    const int i = g * IPT + il;
-    if constexpr (ENDS) S[il] = (DELTA && owns && i < dk && j - dv == i) ? 1.f : 0.f;
-    else if (pieces) S[il] = (i < dk && owns) ? cst[size_t(i) * CW] : 0.f;
-    else S[il] = (i < dk && owns && !fresh) ? st[size_t(i) * dv] : 0.f;
-  }
+  for (int c = 0; c < JPT; ++c)
+#pragma unroll
+    for (int il = 0; il < IPT; ++il) {
+      const int i = g * IPT + il, j = j0 + c * LC;
+      const bool mine = i < dk && j < W;
+      if constexpr (ENDS) S[c][il] = (DELTA && mine && j - dv == i) ? 1.f : 0.f;
+      else if (pieces) S[c][il] = mine ? cst[size_t(i) * CW + j] : 0.f;
+      else S[c][il] = (mine && !fresh) ? st[size_t(i) * dv + j] : 0.f;
+    }
   const float rate = -expf(A.a_log[head]), dtb = A.dt_bias[head];
   const float skip = DELTA ? 0.f : A.d_skip[head];
   const float q_scale = 1.0f / sqrtf(float(dk));
@@ -95,12 +100,12 @@ __global__ void __launch_bounds__(256) gated_state_kernel(StateArgs A) {
       const int e = threadIdx.x + n * 256;
       const int t = e / V, off = e % V;
       const int row = t0 + t < r1 ? t0 + t : r1 - 1;
-      const bool vec = off < 2 * DKP;
-      const int i = off % DKP, jj = cb * CB + (off - 2 * DKP);
+      const bool vec = off < KAT + DKP;
+      const int i = off % DKP, jj = cb * CB + (off - KAT - DKP);
       const bool ok = t < TILE && t0 + t < r1 && (vec ? i < dk : jj < dv);
       const size_t col = size_t(group) * dk + (i < dk ? i : dk - 1);
       const size_t vcol = size_t(head) * dv + ((jj >= 0 && jj < dv) ? jj : 0);
-      const float* src = !vec ? A.v + size_t(row) * A.ldv + vcol : off < DKP ? A.q + size_t(row) * A.ldq + col : A.k + size_t(row) * A.ldk + col;
+      const float* src = !vec ? A.v + size_t(row) * A.ldv + vcol : off < KAT ? A.q + size_t(row) * A.ldq + col : A.k + size_t(row) * A.ldk + col;
       const float val = *src;
       pf[n] = ok ? val : 0.f;
     }
@@ -123,13 +128,15 @@ __global__ void __launch_bounds__(256) gated_state_kernel(StateArgs A) {
     if constexpr (DELTA) {      // the lengths of the staged q and k: sixteen lanes a vector
       __syncthreads();
       const int vec = threadIdx.x / 16, l = threadIdx.x % 16;
-      if (vec < 2 * TILE) {
-        const float* x = &tile[vec / 2][(vec & 1) * DKP];
+      if (ENDS ? vec < TILE : vec < 2 * TILE) {
+        const int t = ENDS ? vec : vec / 2;
+        const bool key = ENDS || (vec & 1);
+        const float* x = &tile[t][key ? KAT : 0];
         float ss = 0.f;
 #pragma unroll
         for (int i = 0; i < DKP / 16; ++i) ss = fmaf(x[l + i * 16], x[l + i * 16], ss);
         ss = group_sum<16>(ss);
-        if (l == 0) tile[vec / 2][V + 2 + (vec & 1)] = (1.0f / sqrtf(ss + 1e-6f)) * ((vec & 1) ? 1.0f : q_scale);
+        if (l == 0) tile[t][V + 2 + (key ? 1 : 0)] = (1.0f / sqrtf(ss + 1e-6f)) * (key ? 1.0f : q_scale);
       }
     }
   };
@@ -143,36 +150,54 @@ __global__ void __launch_bounds__(256) gated_state_kernel(StateArgs A) {
     if (more) request(t0 + TILE);
     for (int t = 0; t < nt; ++t) {
       const float* tv = tile[t];
-      const float keep = tv[V], take = tv[V + 1], vj = tv[2 * DKP + jl];
-      float kd[IPT];
+      const float keep = tv[V], take = tv[V + 1];
+      float kd[IPT], vj[JPT], u[JPT];
 #pragma unroll
-      for (int il = 0; il < IPT; ++il) kd[il] = tv[DKP + g * IPT + il];
-      float u;
+      for (int il = 0; il < IPT; ++il) kd[il] = tv[KAT + g * IPT + il];
+#pragma unroll
+      for (int c = 0; c < JPT; ++c) vj[c] = tv[KAT + DKP + c * LC + jl];
       if constexpr (DELTA) {
         const float fk = tv[V + 3];
-        float sk = 0.f;
 #pragma unroll
-        for (int il = 0; il < IPT; ++il) {
-          S[il] *= keep;
-          sk = fmaf(kd[il], S[il], sk);
+        for (int c = 0; c < JPT; ++c) {
+          float sk = 0.f;
+#pragma unroll
+          for (int il = 0; il < IPT; ++il) {
+            S[c][il] *= keep;
+            sk = fmaf(kd[il], S[c][il], sk);
+          }
+          u[c] = sk;
         }
-        sk = group_sum<G>(sk) * fk;
-        u = take * (vj - sk) * fk;
-      } else {
-        u = take * vj;
 #pragma unroll
-        for (int il = 0; il < IPT; ++il) S[il] *= keep;
+        for (int c = 0; c < JPT; ++c) u[c] = take * (vj[c] - group_sum<G>(u[c]) * fk) * fk;
+      } else {
+#pragma unroll
+        for (int c = 0; c < JPT; ++c) {
+          u[c] = take * vj[c];
+#pragma unroll
+          for (int il = 0; il < IPT; ++il) S[c][il] *= keep;
+        }
         if constexpr (ENDS) decay *= keep;
       }
-      float acc = 0.f;
+      float acc[JPT];
+#pragma unroll
+      for (int c = 0; c < JPT; ++c) acc[c] = 0.f;
 #pragma unroll
       for (int il = 0; il < IPT; ++il) {
-        S[il] = fmaf(kd[il], u, S[il]);
-        if constexpr (!ENDS) acc = fmaf(S[il], tv[g * IPT + il], acc);
+        const float qd = ENDS ? 0.f : tv[g * IPT + il];
+#pragma unroll
+        for (int c = 0; c < JPT; ++c) {
+          S[c][il] = fmaf(kd[il], u[c], S[c][il]);
+          if constexpr (!ENDS) acc[c] = fmaf(S[c][il], qd, acc[c]);
+        }
       }
       if constexpr (!ENDS) {
-        acc = group_sum<G>(acc);
-        if (owns && g == 0) A.o[size_t(t0 + t) * A.ldo + size_t(head) * dv + j] = DELTA ? acc * tv[V + 2] : fmaf(skip, vj, acc);
+#pragma unroll
+        for (int c = 0; c < JPT; ++c) {
+          const float sum = group_sum<G>(acc[c]);
+          const int j = j0 + c * LC;
+          if (j < dv && g == 0) A.o[size_t(t0 + t) * A.ldo + size_t(head) * dv + j] = DELTA ? sum * tv[V + 2] : fmaf(skip, vj[c], sum);
+        }
       }
     }
     __syncthreads();
@@ -181,83 +206,151 @@ __global__ void __launch_bounds__(256) gated_state_kernel(StateArgs A) {
   }
   if constexpr (ENDS) {
 #pragma unroll
-    for (int il = 0; il < IPT; ++il) {
-      const int i = g * IPT + il;
-      if (i < dk && owns) cst[size_t(i) * CW] = S[il];
-    }
+    for (int c = 0; c < JPT; ++c)
+#pragma unroll
+      for (int il = 0; il < IPT; ++il) {
+        const int i = g * IPT + il, j = j0 + c * LC;
+        if (i < dk && j < W) cst[size_t(i) * CW + j] = S[c][il];
+      }
     if (!DELTA && cb == 0 && threadIdx.x == 0)
       A.carry[size_t(A.total_pieces) * A.heads * dk * CW + size_t(piece_place(run0, s, p, A.piece)) * A.heads + head] = decay;
   } else if (last) {
 #pragma unroll
-    for (int il = 0; il < IPT; ++il) {
-      const int i = g * IPT + il;
-      if (i < dk && owns) st[size_t(i) * dv] = S[il];
-    }
+    for (int c = 0; c < JPT; ++c)
+#pragma unroll
+      for (int il = 0; il < IPT; ++il) {
+        const int i = g * IPT + il, j = j0 + c * LC;
+        if (i < dk && j < W) st[size_t(i) * dv + j] = S[c][il];
+      }
   }
 }
 
 // the states that enter a sequence's pieces, walked from its slot (or zero): carry[piece].B <- S, then S <- A S + B.
-// grid (heads * column blocks of 16, sequences); S of these columns in LDS.
+// grid (heads * column blocks of 16, sequences), four lanes a row of S with four columns each; S of these columns in LDS.
+// What a step of the walk reads (the row's part of B, the row of A a stretch at a time) does not depend on the state, so it is
+// requested a stretch ahead (WIDE: sizes in multiples of four, rows of A read 16 bytes at a time; otherwise as it is used).
 constexpr int kPassCols = 16;
-template <bool DELTA>
-__global__ void __launch_bounds__(256) gated_state_pass_kernel(StateArgs A) {
-  extern __shared__ __attribute__((aligned(16))) float cur[];      // [2][dk][kPassCols]
+template <int DKP, bool DELTA, bool WIDE>
+__global__ void __launch_bounds__(DKP * 4) gated_state_pass_kernel(StateArgs A) {
+  constexpr int NB = DKP <= 64 ? 16 : 8;                        // 16-byte pieces of a row of A on their way at once
+  constexpr int STRETCHES = DELTA ? DKP / 4 / NB : 1;
+  __shared__ __attribute__((aligned(16))) float cur[2][DKP][kPassCols];
   const int head = blockIdx.x / A.col_blocks, cb = blockIdx.x % A.col_blocks, s = blockIdx.y;
   const int dk = A.dk, dv = A.dv, CW = DELTA ? dv + dk : dv;
   const int run0 = A.run_start[s], len = A.run_start[s + 1] - run0, slot = A.state_slots[s];
   if (len <= 0 || slot < 0) return;
   const int n = (len + A.piece - 1) / A.piece;
-  const int jl = threadIdx.x % kPassCols, j = cb * kPassCols + jl, jc = j < dv ? j : dv - 1;
+  const int jl = (threadIdx.x % 4) * 4, j0 = cb * kPassCols + jl, i = threadIdx.x / 4, ic = i < dk ? i : dk - 1;
   const bool fresh = A.seq_start[s] == 0;
   const float* st = A.state + (size_t(slot) * A.heads + head) * dk * dv;
   const float* decays = A.carry + size_t(A.total_pieces) * A.heads * dk * CW;
-  float* now = cur;
-  float* next = cur + dk * kPassCols;
-  for (int i = threadIdx.x / kPassCols; i < dk; i += 256 / kPassCols) now[i * kPassCols + jl] = fresh ? 0.f : st[size_t(i) * dv + jc];
-  __syncthreads();
-  for (int p = 0; p < n; ++p) {
-    const size_t place = size_t(piece_place(run0, s, p, A.piece)) * A.heads + head;
-    float* c = A.carry + place * dk * CW;
-    const float keep = !DELTA && p + 1 < n ? decays[place] : 0.f;
-    for (int i = threadIdx.x / kPassCols; i < dk; i += 256 / kPassCols) {
-      float* row = c + size_t(i) * CW;
-      if (p + 1 < n) {
-        float acc = row[jc];
-        if constexpr (DELTA) {
-          const float* a = row + dv;
-#pragma unroll 8
-          for (int m = 0; m < dk; ++m) acc = fmaf(a[m], now[m * kPassCols + jl], acc);
-        } else {
-          acc = fmaf(keep, now[i * kPassCols + jl], acc);
-        }
-        next[i * kPassCols + jl] = acc;
+  auto place = [&](int p) { return size_t(piece_place(run0, s, p, A.piece)) * A.heads + head; };
+  auto row_of = [&](int p) { return A.carry + (place(p) * dk + ic) * CW; };
+  float4 a[NB];
+  float b[4], keep = 0.f;
+  auto request_a = [&](int p, int stretch) {
+    if constexpr (DELTA && WIDE) {
+      const float* src = row_of(p) + dv;
+#pragma unroll
+      for (int q = 0; q < NB; ++q) {
+        const int m = (stretch * NB + q) * 4;
+        a[q] = *reinterpret_cast<const float4*>(src + (m < dk ? m : 0));
       }
-      if (j < dv) row[j] = now[i * kPassCols + jl];      // (a thread reads and writes its own element of B; A is only read)
+    }
+  };
+  auto request_b = [&](int p) {
+    const float* src = row_of(p);
+#pragma unroll
+    for (int c = 0; c < 4; ++c) b[c] = src[j0 + c < dv ? j0 + c : dv - 1];
+    if constexpr (!DELTA) keep = decays[place(p)];
+  };
+  // rows of S beyond dk stay zero: what a row of A multiplies there adds nothing
+#pragma unroll
+  for (int c = 0; c < 4; ++c) {
+    cur[0][i][jl + c] = (fresh || i >= dk || j0 + c >= dv) ? 0.f : st[size_t(i) * dv + j0 + c];
+    cur[1][i][jl + c] = 0.f;
+  }
+  if (n > 1) {
+    request_b(0);
+    request_a(0, 0);
+  }
+  __syncthreads();
+  int now = 0;
+  for (int p = 0; p < n; ++p, now ^= 1) {
+    const float4 mine = *reinterpret_cast<const float4*>(&cur[now][i][jl]);
+    if (p + 1 < n) {
+      float acc[4] = {b[0], b[1], b[2], b[3]};
+      if constexpr (DELTA) {
+        if (p + 2 < n) request_b(p + 1);
+        auto add = [&](float am, int m) {
+          const float4 x = *reinterpret_cast<const float4*>(&cur[now][m][jl]);
+          acc[0] = fmaf(am, x.x, acc[0]);
+          acc[1] = fmaf(am, x.y, acc[1]);
+          acc[2] = fmaf(am, x.z, acc[2]);
+          acc[3] = fmaf(am, x.w, acc[3]);
+        };
+        if constexpr (!WIDE) {
+          const float* src = row_of(p) + dv;
+#pragma unroll 4
+          for (int m = 0; m < dk; ++m) add(src[m], m);
+        } else
+#pragma unroll 1
+        for (int stretch = 0; stretch < STRETCHES; ++stretch) {
+          float4 have[NB];
+#pragma unroll
+          for (int q = 0; q < NB; ++q) have[q] = a[q];
+          if (stretch + 1 < STRETCHES) request_a(p, stretch + 1);
+          else if (p + 2 < n) request_a(p + 1, 0);
+#pragma unroll
+          for (int q = 0; q < NB; ++q) {
+            const int m = (stretch * NB + q) * 4;
+            add(have[q].x, m);
+            add(have[q].y, m + 1);
+            add(have[q].z, m + 2);
+            add(have[q].w, m + 3);
+          }
+        }
+      } else {
+        const float k = keep;
+        if (p + 2 < n) request_b(p + 1);
+        acc[0] = fmaf(k, mine.x, acc[0]);
+        acc[1] = fmaf(k, mine.y, acc[1]);
+        acc[2] = fmaf(k, mine.z, acc[2]);
+        acc[3] = fmaf(k, mine.w, acc[3]);
+      }
+      if (i < dk) *reinterpret_cast<float4*>(&cur[now ^ 1][i][jl]) = float4{acc[0], acc[1], acc[2], acc[3]};
+    }
+    if (i < dk) {      // (a lane reads and writes its own elements of B; A is only read)
+      float* dst = row_of(p);
+      const float v[4] = {mine.x, mine.y, mine.z, mine.w};
+#pragma unroll
+      for (int c = 0; c < 4; ++c)
+        if (j0 + c < dv) dst[j0 + c] = v[c];
     }
     __syncthreads();
-    float* t = now;
-    now = next;
-    next = t;
   }
 }
 
-template <int DKP, int G, int TILE, bool DELTA>
+template <int DKP, int G, int JPT, int TILE, bool DELTA>
 void launch_state(StateArgs A, int S, hipStream_t s) {
-  constexpr int CB = 256 / G;
+  constexpr int CB = JPT * 256 / G;
   if (A.piece == 0) {
     A.pieces_per_seq = 1;
     A.col_blocks = (A.dv + CB - 1) / CB;
-    gated_state_kernel<DKP, G, TILE, DELTA, false><<<dim3(A.heads * A.col_blocks, S), 256, 0, s>>>(A);
+    gated_state_kernel<DKP, G, JPT, TILE, DELTA, false><<<dim3(A.heads * A.col_blocks, S), 256, 0, s>>>(A);
     return;
   }
   const int W = DELTA ? A.dv + A.dk : A.dv;
   StateArgs E = A;
   E.col_blocks = (W + CB - 1) / CB;
-  gated_state_kernel<DKP, G, TILE, DELTA, true><<<dim3(E.heads * E.col_blocks, S * A.pieces_per_seq), 256, 0, s>>>(E);
+  gated_state_kernel<DKP, G, JPT, TILE, DELTA, true><<<dim3(E.heads * E.col_blocks, S * A.pieces_per_seq), 256, 0, s>>>(E);
   E.col_blocks = (A.dv + kPassCols - 1) / kPassCols;
-  gated_state_pass_kernel<DELTA><<<dim3(E.heads * E.col_blocks, S), 256, 2 * sizeof(float) * A.dk * kPassCols, s>>>(E);
+  constexpr int PK = DKP < 64 ? 64 : DKP;
+  const dim3 grid(E.heads * E.col_blocks, S);
+  if (!DELTA || (A.dk % 4 == 0 && A.dv % 4 == 0)) gated_state_pass_kernel<PK, DELTA, true><<<grid, PK * 4, 0, s>>>(E);
+  else gated_state_pass_kernel<PK, DELTA, false><<<grid, PK * 4, 0, s>>>(E);
   E.col_blocks = (A.dv + CB - 1) / CB;
-  gated_state_kernel<DKP, G, TILE, DELTA, false><<<dim3(E.heads * E.col_blocks, S * A.pieces_per_seq), 256, 0, s>>>(E);
+  gated_state_kernel<DKP, G, JPT, TILE, DELTA, false><<<dim3(E.heads * E.col_blocks, S * A.pieces_per_seq), 256, 0, s>>>(E);
 }
 
 }  // namespace kvcm
@@ -297,16 +390,18 @@ int kvcm_gated_state(const float* q, int ldq, const float* k, int ldk, const flo
     A.total_pieces = T / piece + S + 1;
   }
   KVCM_REQUIRE(static_cast<long long>(S) * A.pieces_per_seq <= 65535, "gated_state: too many sequences and pieces for one launch");
-#define KVCM_STATE(DKP, G, TILE)                                    \
+#define KVCM_STATE(DKP, G, JPT, TILE)                               \
   {                                                                 \
-    if (delta) launch_state<DKP, G, TILE, true>(A, S, s);           \
-    else launch_state<DKP, G, TILE, false>(A, S, s);                \
+    if (delta) launch_state<DKP, G, JPT, TILE, true>(A, S, s);      \
+    else launch_state<DKP, G, JPT, TILE, false>(A, S, s);           \
   }
-  if (dk <= 16) KVCM_STATE(16, 4, 8)
-  else if (dk <= 32) KVCM_STATE(32, 8, 8)
-  else if (dk <= 64) KVCM_STATE(64, 8, 8)
-  else if (dk <= 128) KVCM_STATE(128, 16, 8)
-  else KVCM_STATE(256, 16, 4)
+  // steps of single rows spread a state over as many workgroups as they can; runs of rows give a lane more of it to keep
+  const bool rows = max_run >= 16;
+  if (dk <= 16) KVCM_STATE(16, 4, 1, 8)
+  else if (dk <= 32) KVCM_STATE(32, 8, 1, 8)
+  else if (dk <= 64) { if (rows) KVCM_STATE(64, 4, 1, 8) else KVCM_STATE(64, 8, 1, 8) }
+  else if (dk <= 128) { if (rows) KVCM_STATE(128, 8, 2, 8) else KVCM_STATE(128, 16, 1, 8) }
+  else KVCM_STATE(256, 16, 1, 4)
 #undef KVCM_STATE
   return launch_status("gated_state");
 }

@@ -201,10 +201,10 @@ __global__ void __launch_bounds__(256)
     head_norm_gate_kernel(const float* __restrict__ o, int ldo, const float* __restrict__ g, int ldg,
                           const float* __restrict__ w, TO* __restrict__ out, int ldout, long long items, int heads,
                           int d, float eps, int gate_silu) {
-  const long long item = static_cast<long long>(blockIdx.x) * (256 / kWave) + threadIdx.x / kWave;
-  if (item >= items) return;
+  const unsigned item = blockIdx.x * (256 / kWave) + threadIdx.x / kWave;      // (items fit 32 bits: a division of 64-bit numbers costs more than the norm)
+  if (item >= static_cast<unsigned long long>(items)) return;
   const int lane = threadIdx.x % kWave;
-  const int row = static_cast<int>(item / heads), head = static_cast<int>(item % heads);
+  const int row = static_cast<int>(item / unsigned(heads)), head = static_cast<int>(item % unsigned(heads));
   const float* orow = o + size_t(row) * ldo + size_t(head) * d;
   const float* grow = g + size_t(row) * ldg + size_t(head) * d;
   float ss = 0.f;
@@ -269,7 +269,7 @@ int kvcm_head_norm_gate(const float* o, int ldo, const float* g, int ldg, const 
   KVCM_REQUIRE(ldo >= heads * d && ldg >= heads * d && ldout >= heads * d, "head_norm_gate: row strides too small");
   const long long items = static_cast<long long>(T) * heads;
   const long long blocks = (items + 3) / 4;
-  KVCM_REQUIRE(blocks < (1ll << 31), "head_norm_gate: too many rows");
+  KVCM_REQUIRE(items < (1ll << 31), "head_norm_gate: too many rows");
   if (out_dtype == kF32)
     head_norm_gate_kernel<float><<<static_cast<unsigned>(blocks), 256, 0, s>>>(o, ldo, g, ldg, w, static_cast<float*>(out),
                                                                                 ldout, items, heads, d, eps, gate_silu);

@@ -144,11 +144,11 @@ __global__ void __launch_bounds__(256)
                            const int* __restrict__ positions, float temp_coef,
                            int temp_every, int values_are_keys, const int* __restrict__ slots, T* __restrict__ q_out, int ldq,
                            T* __restrict__ kcache, T* __restrict__ vcache, long long items, int nh, int nkv, int d, int dv, int B) {
-  const long long item = static_cast<long long>(blockIdx.x) * (256 / kWave) + threadIdx.x / kWave;
-  if (item >= items) return;
+  const unsigned item = blockIdx.x * (256 / kWave) + threadIdx.x / kWave;      // (items fit 32 bits)
+  if (item >= static_cast<unsigned long long>(items)) return;
   const int lane = threadIdx.x % kWave;
   const int per_row = nh + nkv + (values_are_keys ? 0 : nkv);
-  const int row = static_cast<int>(item / per_row), part = static_cast<int>(item % per_row);
+  const int row = static_cast<int>(item / unsigned(per_row)), part = static_cast<int>(item % unsigned(per_row));
   const float* r = src + size_t(row) * ld;
   const int slot = slots ? slots[row] : -1;
   if (part >= nh + nkv) {      // a value head of the projection's own
@@ -173,11 +173,16 @@ __global__ void __launch_bounds__(256)
     const float2 a = cs[halves ? (second ? i - hr : i) : i / 2];
     return second ? __fmaf_rn(x, a.x, __fmul_rn(y, a.y)) : __fmaf_rn(x, a.x, -__fmul_rn(y, a.y));
   };
+  constexpr int kHeld = 4;      // entries a lane keeps: heads of up to 256 are read and turned once
+  float held[kHeld];
+#pragma unroll
+  for (int j = 0; j < kHeld; ++j) held[j] = lane + j * kWave < d ? entry(lane + j * kWave) : 0.f;
+  auto turned = [&](int i) { return i < kHeld * kWave ? (i < 2 * kWave ? (i < kWave ? held[0] : held[1]) : (i < 3 * kWave ? held[2] : held[3])) : entry(i); };
   float inv = 1.f;
   if (w || plain_norm) {
     float ss = 0.f;
     for (int i = lane; i < d; i += kWave) {
-      const float x = entry(i);
+      const float x = turned(i);
       ss = fmaf(x, x, ss);
     }
     inv = 1.0f / sqrtf(wave_sum(ss) / float(d) + eps);
@@ -186,14 +191,14 @@ __global__ void __launch_bounds__(256)
     float temp = 1.f;
     if (temp_every > 0) temp = fmaf(temp_coef, logf(float((positions[row] + 1) / temp_every + 1)), 1.0f);
     for (int i = lane; i < d; i += kWave) {
-      const float x = entry(i) * inv;
+      const float x = turned(i) * inv;
       store_f(q_out + size_t(row) * ldq + at + i, (w ? x * w[i] : x) * temp);
     }
     return;
   }
   const int head = part - nh;
   for (int i = lane; i < d; i += kWave) {
-    const float x = entry(i) * inv;
+    const float x = turned(i) * inv;
     store_f(kcache + ((size_t(slot / B) * nkv + head) * B + slot % B) * d + i, w ? x * w[i] : x);
     if (values_are_keys) store_f(vcache + ((size_t(slot / B) * nkv + head) * dv + i) * B + slot % B, projected(i));
   }
@@ -249,7 +254,7 @@ int kvcm_head_norm_store(const float* src, int ld, const float* bias, const floa
   KVCM_REQUIRE(!slots || (kcache && vcache), "head_norm_store: slots without pages");
   const long long items = static_cast<long long>(T) * (nh + nkv + (values_are_keys ? 0 : nkv));
   const long long blocks = (items + 3) / 4;
-  KVCM_REQUIRE(blocks < (1ll << 31), "head_norm_store: too many rows");
+  KVCM_REQUIRE(items < (1ll << 31), "head_norm_store: too many rows");
   if (dtype == kF32)
     head_norm_store_kernel<float><<<static_cast<unsigned>(blocks), 256, 0, s>>>(
         src, ld, bias, wq, wk, eps, plain_norm, reinterpret_cast<const float2*>(cos_sin), rot, halves, positions, temp_coef, temp_every, values_are_keys, slots, static_cast<float*>(q_out), ldq,

@@ -62,6 +62,67 @@ __global__ void __launch_bounds__(256)
   store_f(dst, y);
 }
 
+// The same for steps with runs of rows: a thread walks kConvRows consecutive rows of its channel with the taps' inputs in
+// registers, so that an input is read once instead of once per tap, and the weights once for all rows.  The operations of a
+// row are those of the kernel above, in the same order.
+constexpr int kConvRows = 16;
+template <class TO, int TAPS>
+__global__ void __launch_bounds__(256)
+    short_conv_rows_kernel(const float* __restrict__ in, int ld_in, const float* __restrict__ bias_in,
+                           const float* __restrict__ w, const float* __restrict__ bias_out, const float* __restrict__ state,
+                           TO* __restrict__ out, int ld_out, const int* __restrict__ row_seq, const int* __restrict__ positions,
+                           const int* __restrict__ ctx_lens, const int* __restrict__ run_start, const int* __restrict__ seq_start,
+                           const int* __restrict__ state_slots, int T, int C, int act) {
+  const int c = blockIdx.x * 256 + threadIdx.x;
+  const int first = blockIdx.y * kConvRows, end = first + kConvRows < T ? first + kConvRows : T;
+  if (c >= C) return;
+  const float bi = bias_in ? bias_in[c] : 0.f, bo = bias_out ? bias_out[c] : 0.f;
+  float wt[TAPS], seen[TAPS];
+#pragma unroll
+  for (int j = 0; j < TAPS; ++j) wt[j] = w[size_t(c) * TAPS + j];
+  float x[kConvRows];
+#pragma unroll
+  for (int r = 0; r < kConvRows; ++r) {      // all on their way together
+    const int row = first + r < end ? first + r : end - 1;
+    x[r] = in[size_t(row) * ld_in + c];
+  }
+  int s_before = -1;
+#pragma unroll
+  for (int r = 0; r < kConvRows; ++r) {
+    const int row = first + r;
+    if (row >= end) break;
+    TO* dst = out + size_t(row) * ld_out + c;
+    if (ctx_lens[row] <= 0) {      // a padding row
+      store_f(dst, 0.f);
+      s_before = -1;
+      continue;
+    }
+    const int s = row_seq[row];
+    if (s != s_before) {      // the block's first row, or another sequence's: the inputs before this row
+      const int p = positions[row], p0 = seq_start[s], r0 = run_start[s], slot = state_slots[s];
+      const float* st = slot >= 0 ? state + (size_t(slot) * (TAPS - 1)) * C + c : nullptr;
+#pragma unroll
+      for (int j = 0; j < TAPS - 1; ++j) {
+        const int t = p - (TAPS - 1) + j;
+        float u = 0.f;
+        if (t >= p0) u = in[size_t(r0 + (t - p0)) * ld_in + c] + bi;
+        else if (t >= 0 && st) u = st[size_t(t - (p0 - (TAPS - 1))) * C];
+        seen[j] = u;
+      }
+      s_before = s;
+    }
+    seen[TAPS - 1] = x[r] + bi;
+    float y = 0.f;
+#pragma unroll
+    for (int j = 0; j < TAPS; ++j) y = fmaf(wt[j], seen[j], y);
+#pragma unroll
+    for (int j = 0; j < TAPS - 1; ++j) seen[j] = seen[j + 1];
+    if (bias_out) y += bo;
+    if (act == 1) y = y / (1.0f + expf(-y));
+    store_f(dst, y);
+  }
+}
+
 // state[slot][k][c] <- the input at position end - (taps-1) + k, k = 0 .. taps-2
 __global__ void __launch_bounds__(256)
     short_conv_state_kernel(const float* __restrict__ in, int ld_in, const float* __restrict__ bias_in,
@@ -109,6 +170,17 @@ int kvcm_short_conv(const float* in, int ld_in, const float* bias_in, const floa
   KVCM_REQUIRE(ld_in >= C && ld_out >= C, "short_conv: row strides too small");
   KVCM_REQUIRE(T <= 65535, "short_conv: too many rows for one launch (%d)", T);
   KVCM_REQUIRE(act == 0 || act == 1, "short_conv: unknown activation %d", act);
+  KVCM_REQUIRE(out_dtype == kF32 || out_dtype == kBF16, "short_conv: unknown output dtype %d", out_dtype);
+  if (!update_state && T >= kConvRows && taps >= 2 && taps <= 4) {
+    const dim3 grid((C + 255) / 256, (T + kConvRows - 1) / kConvRows);
+#define KVCM_CONV_ROWS(TO, TAPS)                                                                                            \
+  short_conv_rows_kernel<TO, TAPS><<<grid, 256, 0, s>>>(in, ld_in, bias_in, w, bias_out, state, static_cast<TO*>(out), ld_out, \
+                                                        row_seq, positions, ctx_lens, run_start, seq_start, state_slots, T, C, act)
+    if (out_dtype == kF32) { if (taps == 2) KVCM_CONV_ROWS(float, 2); else if (taps == 3) KVCM_CONV_ROWS(float, 3); else KVCM_CONV_ROWS(float, 4); }
+    else { if (taps == 2) KVCM_CONV_ROWS(bf16_t, 2); else if (taps == 3) KVCM_CONV_ROWS(bf16_t, 3); else KVCM_CONV_ROWS(bf16_t, 4); }
+#undef KVCM_CONV_ROWS
+    return launch_status("short_conv");
+  }
   const dim3 grid((C + 255) / 256, T);
   if (out_dtype == kF32)
     short_conv_kernel<float><<<grid, 256, 0, s>>>(in, ld_in, bias_in, w, bias_out, state, static_cast<float*>(out), ld_out,

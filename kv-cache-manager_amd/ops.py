@@ -1794,12 +1794,16 @@ def group_norm_gate(y, z, weight, out, groups, size, eps):
     return out
 
 
-GATED_STATE_PIECE = 128      # rows of a piece when long runs are walked in pieces
+def gated_state_piece(dk):
+    """Rows of a piece when long runs are walked in pieces.  Measured on 2,048 rows of 32 heads (the three launches together,
+    delta rule): 64 x 64 states 202 / 178 / 226 us with pieces of 64 / 128 / 256 rows, 128 x 128 states 625 / 473 / 432 us
+    (walked without pieces: 923 and 1,275 us)."""
+    return 128 if dk <= 64 else 256
 
 
-def gated_state_carry_floats(rows, seqs, heads, dk, dv, delta, piece=GATED_STATE_PIECE):
+def gated_state_carry_floats(rows, seqs, heads, dk, dv, delta, piece=None):
     """32-bit values of scratch that ``gated_state`` needs to walk a step of this shape in pieces."""
-    return int(lib().kvcm_gated_state_carry_floats(rows, seqs, heads, dk, dv, 1 if delta else 0, piece))
+    return int(lib().kvcm_gated_state_carry_floats(rows, seqs, heads, dk, dv, 1 if delta else 0, piece or gated_state_piece(dk)))
 
 
 def gated_state(q, k, v, a, dt_bias, a_log, o, state, step, heads, groups, dk, dv, b=None, d_skip=None, carry=None, piece=None):
@@ -1819,7 +1823,7 @@ def gated_state(q, k, v, a, dt_bias, a_log, o, state, step, heads, groups, dk, d
         _f32(t, n, heads)
     _need(state.dtype == torch.float32 and state.is_contiguous() and state.is_cuda and tuple(state.shape[1:]) == (heads, dk, dv),
           "state must be float32 [slots, heads, dk, dv]")
-    piece = (GATED_STATE_PIECE if piece is None else int(piece)) if carry is not None else 0
+    piece = int(piece or gated_state_piece(dk)) if carry is not None else 0
     _f32(carry, "carry")
     _call("kvcm_gated_state", _ptr(q), q.stride(0), _ptr(k), k.stride(0), _ptr(v), v.stride(0), _ptr(a), a.stride(0), _ptr(b),
           b.stride(0) if delta else 0, _ptr(dt_bias), _ptr(a_log), _ptr(d_skip), 1 if delta else 0, _ptr(o), o.stride(0), _ptr(state),

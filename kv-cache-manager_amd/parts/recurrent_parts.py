@@ -222,7 +222,7 @@ class _ConvStateMixer(EndsMixer):
     def carry(self, step, heads, dk, dv, delta):
         """Scratch for walking long runs in pieces, sized for the engine's largest step; None for steps of short runs."""
         ops = self.ctx.ops
-        if step.max_run < 4 * ops.GATED_STATE_PIECE:
+        if step.max_run < 4 * ops.gated_state_piece(dk):
             return None
         lim = step.limits
         rows, seqs = max(step.rows, lim.max_tokens if lim else 0), max(step.seqs, lim.max_seqs if lim else 0)
