@@ -5,3 +5,4 @@ from . import furapel  # noqa: F401
 from . import fisesun  # noqa: F401
 from . import betirax  # noqa: F401
 from . import vugotar  # noqa: F401
+from . import zalunex  # noqa: F401

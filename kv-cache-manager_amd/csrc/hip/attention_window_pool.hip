@@ -9,8 +9,9 @@
 //   and all of them share one softmax; score = (q . k) * scale_h with a factor per query head, and with a cap c > 0
 //   score <- c tanh(score / c); then, with a slope per query head, score <- score - slope_h * (i - j) for token j (a bias
 //   that grows with the distance; not offered together with pooled blocks, which have no one distance).  The output may be
-//   multiplied element by element with sigmoid(gate) (32-bit gate logits of the output's shape) before it is stored, and by a
-//   constant factor.  With a sink, one is added to the softmax's denominator: a key of score 0 that has no value.
+//   multiplied with sigmoid(gate) before it is stored, element by element (32-bit gate logits of the output's shape) or head by
+//   head (one logit each), and by a constant factor.  With a sink, one summand more joins the softmax's denominator: a key
+//   without a value whose score is 0, or a number per query head that neither scale nor cap touches.
 //
 // Pages: keys [pages, kv_heads, B, d], values transposed [pages, kv_heads, dv, B] (as the other
 // attentions of this library keep them).  Pooled entries are 32-bit and live with the page that holds
@@ -267,7 +268,7 @@ __global__ void __launch_bounds__(kWpWaves* kWave)
                                  const int* __restrict__ ctx_lens, const float* __restrict__ head_scale,
                                  const float* __restrict__ dist_slope, const float* __restrict__ gate, int ldg,
                                  int nh, int nkv, int d, int dv, int B, float scale, int window, int P, int E, int keep_first,
-                                 float softcap, int chunk, int sink, float out_scale) {
+                                 float softcap, int chunk, int sink, const float* __restrict__ sink_logit, int gate_heads, float out_scale) {
   extern __shared__ float lds[];      // [d] q * scale * head_scale[h]; [waves][64] probabilities; [waves][dv + 2] results
   constexpr int N = RowPiece<T>::N, COLS = kWpMaxValueDim / kWave;
   const int wave = threadIdx.x / kWave, lane = threadIdx.x % kWave;
@@ -410,22 +411,24 @@ __global__ void __launch_bounds__(kWpWaves* kWave)
     mine[dv + 1] = l;
   }
   __syncthreads();
-  float mm = sink ? 0.f : -INFINITY;
+  const float sl = sink_logit ? sink_logit[head] : 0.f;
+  float mm = sink ? sl : -INFINITY;
 #pragma unroll
   for (int w = 0; w < kWpWaves; ++w) mm = fmaxf(mm, merge[w * (dv + 2) + dv]);
-  float wgt[kWpWaves], ll = sink ? expf(-mm) : 0.f;
+  float wgt[kWpWaves], ll = sink ? expf(sl - mm) : 0.f;
 #pragma unroll
   for (int w = 0; w < kWpWaves; ++w) {
     const float mw = merge[w * (dv + 2) + dv];
     wgt[w] = mw == -INFINITY ? 0.f : expf(mw - mm);
     ll = fmaf(merge[w * (dv + 2) + dv + 1], wgt[w], ll);
   }
+  const float* gr = gate ? gate + size_t(row) * ldg + (gate_heads ? head : head * dv) : nullptr;
   for (int cc = threadIdx.x; cc < dv; cc += kWpWaves * kWave) {
     float acc = 0.f;
 #pragma unroll
     for (int w = 0; w < kWpWaves; ++w) acc = fmaf(merge[w * (dv + 2) + cc], wgt[w], acc);
     float res = acc / ll * out_scale;
-    if (gate) res *= 1.0f / (1.0f + expf(-gate[size_t(row) * ldg + size_t(head) * dv + cc]));      // a gate per element of the output
+    if (gate) res *= 1.0f / (1.0f + expf(-gr[gate_heads ? 0 : cc]));      // a gate per element of the output, or one per head
     store_f(orow + cc, res);
   }
 }
@@ -528,7 +531,7 @@ int kvcm_attention_window_pool(const void* q, int dtype, int ldq, void* out, int
                                const float* pk, const float* pv, const int* tables, int table_stride, const int* row_seq,
                                const int* ctx_lens, const float* head_scale, const float* dist_slope, const float* gate, int ldg,
                                int T, int nh, int nkv, int d, int dv, int B, float scale, int window, int P, int E, int keep_first,
-                               float softcap, int chunk, int sink, float out_scale, hipStream_t s) {
+                               float softcap, int chunk, int sink, const float* __restrict__ sink_logit, int gate_heads, float out_scale, hipStream_t s) {
   if (T == 0) return 0;
   KVCM_REQUIRE(T > 0 && nh > 0 && nkv > 0 && B > 0 && d > 0, "attention_window_pool: bad sizes T=%d heads=%d kv_heads=%d", T, nh, nkv);
   KVCM_REQUIRE(nh % nkv == 0, "attention_window_pool: %d query heads are not a multiple of %d kv heads", nh, nkv);
@@ -539,7 +542,7 @@ int kvcm_attention_window_pool(const void* q, int dtype, int ldq, void* out, int
   KVCM_REQUIRE(P == 0 || (pk && pv && E == (B + P - 1) / P), "attention_window_pool: pooled blocks need their entries");
   KVCM_REQUIRE(keep_first >= 0 && softcap >= 0.f, "attention_window_pool: negative count of kept tokens or score cap");
   KVCM_REQUIRE(!dist_slope || P == 0, "attention_window_pool: a distance bias beside pooled blocks is not supported");
-  KVCM_REQUIRE(!gate || ldg >= nh * dv, "attention_window_pool: the gate's rows are too short");
+  KVCM_REQUIRE(!gate || ldg >= (gate_heads ? nh : nh * dv), "attention_window_pool: the gate's rows are too short");
   KVCM_REQUIRE(chunk >= 0 && (chunk == 0 || (window == 0 && P == 0 && keep_first == 0)),
                "attention_window_pool: a chunk beside a window, pooled blocks or kept first tokens is not supported");
   const long long blocks = static_cast<long long>(T) * nh;
@@ -549,12 +552,12 @@ int kvcm_attention_window_pool(const void* q, int dtype, int ldq, void* out, int
     attention_window_pool_kernel<float><<<static_cast<unsigned>(blocks), kWpWaves * kWave, lds, s>>>(
         static_cast<const float*>(q), ldq, static_cast<float*>(out), ldo, static_cast<const float*>(kcache),
         static_cast<const float*>(vcache), pk, pv, tables, table_stride, row_seq, ctx_lens, head_scale, dist_slope, gate,
-        ldg, nh, nkv, d, dv, B, scale, window, P, E, keep_first, softcap, chunk, sink, out_scale);
+        ldg, nh, nkv, d, dv, B, scale, window, P, E, keep_first, softcap, chunk, sink, sink_logit, gate_heads, out_scale);
   else if (dtype == kBF16)
     attention_window_pool_kernel<bf16_t><<<static_cast<unsigned>(blocks), kWpWaves * kWave, lds, s>>>(
         static_cast<const bf16_t*>(q), ldq, static_cast<bf16_t*>(out), ldo, static_cast<const bf16_t*>(kcache),
         static_cast<const bf16_t*>(vcache), pk, pv, tables, table_stride, row_seq, ctx_lens, head_scale, dist_slope, gate,
-        ldg, nh, nkv, d, dv, B, scale, window, P, E, keep_first, softcap, chunk, sink, out_scale);
+        ldg, nh, nkv, d, dv, B, scale, window, P, E, keep_first, softcap, chunk, sink, sink_logit, gate_heads, out_scale);
   else KVCM_REQUIRE(false, "attention_window_pool: unknown dtype %d", dtype);
   return launch_status("attention_window_pool");
 }

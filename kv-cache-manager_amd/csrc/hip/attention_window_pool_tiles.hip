@@ -10,8 +10,9 @@
 // keep_first tokens of a sequence may stay visible beyond the window (chunks of their own, from token 0), and the
 // scores may be capped, score <- c tanh(score / c), and a bias that grows with the distance may be taken off them,
 // score <- score - slope_h * (i - j) with a slope per query head (tokens only: not beside pooled blocks); the output may be
-// multiplied element by element with sigmoid(gate) before it is stored, and by a constant factor.  With a chunk size in the
-// window's place a row sees its own chunk of positions only; with a sink, one is added to the softmax's denominator.
+// multiplied with sigmoid(gate) before it is stored, element by element or head by head, and by a constant factor.  With a
+// chunk size in the window's place a row sees its own chunk of positions only; with a sink, a key without a value (score 0, or
+// a number per query head) joins the softmax's denominator.
 // bfloat16 storage only; sizes d and dv in multiples of 8, pages whose size is a multiple of 8 and divides 64.
 #include <cfloat>
 
@@ -40,7 +41,7 @@ __global__ void __launch_bounds__(256)
                                        const int* __restrict__ seq_start, const float* __restrict__ head_scale,
                                        const float* __restrict__ dist_slope, const float* __restrict__ gate, int ldg, int tiles_per_seq,
                                        int nh, int nkv, int d, int dv, int B, float scale, int window, int P, int E,
-                                       int keep_first, float softcap, int chunk, int sink, float out_scale) {
+                                       int keep_first, float softcap, int chunk, int sink, const float* __restrict__ sink_logit, int gate_heads, float out_scale) {
   constexpr int KP = DP + 8, KS = DP / 32, DVP = DVT * 16;
   __shared__ __attribute__((aligned(16))) uint16_t Ks[kChunk][KP];
   __shared__ __attribute__((aligned(16))) uint16_t Vt[DVP][kVtPitch];
@@ -241,24 +242,26 @@ __global__ void __launch_bounds__(256)
       }
     }
   }
+  const float sl2 = sink_logit ? sink_logit[head] * kLog2e : 0.f;
 #pragma unroll
   for (int i = 0; i < 4; ++i) {
     float l = group_sum<16>(lsum[i]), factor = out_scale;
-    if (sink) {      // a score of 0 joins the denominator (scores are in units of log 2 here too)
-      const float m_all = fmaxf(m[i], 0.f);
+    if (sink) {      // the head's sink (a score of 0 without a number of its own) joins the denominator, in units of log 2 too
+      const float m_all = fmaxf(m[i], sl2);
       const float keep = __builtin_amdgcn_exp2f(m[i] - m_all);
-      l = l * keep + __builtin_amdgcn_exp2f(-m_all);
+      l = l * keep + __builtin_amdgcn_exp2f(sl2 - m_all);
       factor *= keep;
     }
     const int row = wave * 16 + quad * 4 + i;
     if (row < nrows) {
-      const float inv = factor / l;
+      float inv = factor / l;
+      if (gate && gate_heads) inv *= 1.0f / (1.0f + expf(-gate[size_t(r0 + row) * ldg + head]));      // one gate per head
 #pragma unroll
       for (int vt = 0; vt < DVT; ++vt) {
         const int cc = vt * 16 + col;
         if (cc < dv) {
           float res = o[vt][i] * inv;
-          if (gate) res *= 1.0f / (1.0f + expf(-gate[size_t(r0 + row) * ldg + size_t(head) * dv + cc]));      // a gate per element
+          if (gate && !gate_heads) res *= 1.0f / (1.0f + expf(-gate[size_t(r0 + row) * ldg + size_t(head) * dv + cc]));      // a gate per element
           out[size_t(r0 + row) * ldo + size_t(head) * dv + cc] = float_to_bf16_bits(res);
         }
       }
@@ -271,11 +274,11 @@ int launch_tiles(int dvt, dim3 grid, hipStream_t s, const uint16_t* q, int ldq, 
                  const uint16_t* vc, const float* pk, const float* pv, const int* tables, int table_stride, const int* run_start,
                  const int* seq_start, const float* head_scale, const float* dist_slope, const float* gate, int ldg, int tiles_per_seq,
                  int nh, int nkv, int d, int dv, int B, float scale, int window, int P, int E, int keep_first, float softcap,
-                 int chunk, int sink, float out_scale) {
+                 int chunk, int sink, const float* __restrict__ sink_logit, int gate_heads, float out_scale) {
 #define KVCM_TILES(DVT)                                                                                                     \
   attention_window_pool_tiles_kernel<DP, DVT><<<grid, 256, 0, s>>>(q, ldq, out, ldo, kc, vc, pk, pv, tables, table_stride,   \
                                                                    run_start, seq_start, head_scale, dist_slope, gate, ldg, tiles_per_seq, \
-                                                                   nh, nkv, d, dv, B, scale, window, P, E, keep_first, softcap, chunk, sink, out_scale)
+                                                                   nh, nkv, d, dv, B, scale, window, P, E, keep_first, softcap, chunk, sink, sink_logit, gate_heads, out_scale)
   if (dvt <= 2) KVCM_TILES(2);
   else if (dvt <= 4) KVCM_TILES(4);
   else if (dvt <= 8) KVCM_TILES(8);
@@ -299,7 +302,7 @@ int kvcm_attention_window_pool_tiles(const void* q, int ldq, void* out, int ldo,
                                      const float* pk, const float* pv, const int* tables, int table_stride,
                                      const int* run_start, const int* seq_start, const float* head_scale, const float* dist_slope,
                                      const float* gate, int ldg, int S, int max_run, int nh, int nkv, int d, int dv, int B, float scale, int window, int P,
-                                     int E, int keep_first, float softcap, int chunk, int sink, float out_scale, hipStream_t s) {
+                                     int E, int keep_first, float softcap, int chunk, int sink, const float* __restrict__ sink_logit, int gate_heads, float out_scale, hipStream_t s) {
   if (S == 0 || max_run == 0) return 0;
   KVCM_REQUIRE(S > 0 && max_run > 0 && nh > 0 && nkv > 0 && nh % nkv == 0, "attention_window_pool_tiles: bad sizes");
   KVCM_REQUIRE(kvcm_attention_window_pool_tiles_supported(d, dv, B),
@@ -311,7 +314,7 @@ int kvcm_attention_window_pool_tiles(const void* q, int ldq, void* out, int ldo,
   KVCM_REQUIRE(P == 0 || d % 8 == 0, "attention_window_pool_tiles: pooled keys are read eight at a time");
   KVCM_REQUIRE(keep_first >= 0 && softcap >= 0.f, "attention_window_pool_tiles: negative count of kept tokens or score cap");
   KVCM_REQUIRE(!dist_slope || P == 0, "attention_window_pool_tiles: a distance bias beside pooled blocks is not supported");
-  KVCM_REQUIRE(!gate || ldg >= nh * dv, "attention_window_pool_tiles: the gate's rows are too short");
+  KVCM_REQUIRE(!gate || ldg >= (gate_heads ? nh : nh * dv), "attention_window_pool_tiles: the gate's rows are too short");
   KVCM_REQUIRE(chunk >= 0 && (chunk == 0 || (window == 0 && P == 0 && keep_first == 0)),
                "attention_window_pool_tiles: a chunk beside a window, pooled blocks or kept first tokens is not supported");
   const int tiles_per_seq = (max_run + kTileRows - 1) / kTileRows;
@@ -324,12 +327,12 @@ int kvcm_attention_window_pool_tiles(const void* q, int ldq, void* out, int ldo,
   const uint16_t* vc = static_cast<const uint16_t*>(vcache);
   if (d <= 32)
     return launch_tiles<32>(dvt, grid, s, qq, ldq, oo, ldo, kc, vc, pk, pv, tables, table_stride, run_start, seq_start, head_scale,
-                            dist_slope, gate, ldg, tiles_per_seq, nh, nkv, d, dv, B, scale, window, P, E, keep_first, softcap, chunk, sink, out_scale);
+                            dist_slope, gate, ldg, tiles_per_seq, nh, nkv, d, dv, B, scale, window, P, E, keep_first, softcap, chunk, sink, sink_logit, gate_heads, out_scale);
   if (d <= 64)
     return launch_tiles<64>(dvt, grid, s, qq, ldq, oo, ldo, kc, vc, pk, pv, tables, table_stride, run_start, seq_start, head_scale,
-                            dist_slope, gate, ldg, tiles_per_seq, nh, nkv, d, dv, B, scale, window, P, E, keep_first, softcap, chunk, sink, out_scale);
+                            dist_slope, gate, ldg, tiles_per_seq, nh, nkv, d, dv, B, scale, window, P, E, keep_first, softcap, chunk, sink, sink_logit, gate_heads, out_scale);
   return launch_tiles<128>(dvt, grid, s, qq, ldq, oo, ldo, kc, vc, pk, pv, tables, table_stride, run_start, seq_start, head_scale,
-                           dist_slope, gate, ldg, tiles_per_seq, nh, nkv, d, dv, B, scale, window, P, E, keep_first, softcap, chunk, sink, out_scale);
+                           dist_slope, gate, ldg, tiles_per_seq, nh, nkv, d, dv, B, scale, window, P, E, keep_first, softcap, chunk, sink, sink_logit, gate_heads, out_scale);
 }
 
 }  // extern "C"

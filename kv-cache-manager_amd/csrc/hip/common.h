@@ -45,6 +45,22 @@ template <> __device__ __forceinline__ float silu<bf16_t>(float x) {
   return x * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-1.44269504088896341f * x));
 }
 
+// Activations of feed-forwards by number, in 32-bit: 0 silu, 1 relu, 2 gelu by tanh (0.5 z (1 + tanh(sqrt(2/pi) (z +
+// 0.044715 z^3)))), 3 gelu by the error function (z times the normal distribution's function of z).
+__device__ __forceinline__ float ff_activation(int act, float z) {
+  if (act == 1) return fmaxf(z, 0.f);
+  if (act == 2) return 0.5f * z * (1.0f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
+  if (act == 3) return 0.5f * z * (1.0f + erff(z * 0.70710678118654752f));
+  return z / (1.0f + expf(-z));
+}
+
+// A gate with limits: g = min(gate, limit), u = up held within [-limit, limit], g / (1 + exp(-1.702 g)) * (u + 1).
+constexpr float kClampedGateSlope = 1.702f;
+template <class T> __device__ __forceinline__ float clamped_gate(float gate, float up, float limit) {
+  const float g = fminf(gate, limit), u = fminf(fmaxf(up, -limit), limit);
+  return silu<T>(kClampedGateSlope * g) * (1.0f / kClampedGateSlope) * (u + 1.0f);
+}
+
 // (a, b) rotated by the angle whose cosine and sine are given.  One explicit sequence of
 // operations, shared by every kernel that rotates, so that all of them give the same bits.
 __device__ __forceinline__ void rotate_pair(float& a, float& b, float cs, float sn) {

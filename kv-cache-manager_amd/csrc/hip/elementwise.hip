@@ -429,7 +429,8 @@ __global__ void add_residual_kernel(float* __restrict__ x, const T* __restrict__
 // ---------------------------------------------------------------- embedding with a factor
 template <class TW>
 __global__ void embed_scaled_kernel(const int* __restrict__ ids, const TW* __restrict__ table, float* __restrict__ x,
-                                    int H, int V, float factor) {
+                                    int H, int V, float factor, const int* __restrict__ positions, const TW* __restrict__ pos_table,
+                                    int P) {
   const int t = blockIdx.x;
   const int id = ids[t];
   float* dst = x + size_t(t) * H;
@@ -438,16 +439,22 @@ __global__ void embed_scaled_kernel(const int* __restrict__ ids, const TW* __res
     return;
   }
   const TW* src = table + size_t(id) * H;
+  const int p = pos_table ? positions[t] : -1;      // a learned vector per position, unscaled (no position beyond the table gets here)
+  if (p >= 0 && p < P) {
+    const TW* at = pos_table + size_t(p) * H;
+    for (int i = threadIdx.x; i < H; i += blockDim.x) dst[i] = fmaf(load_f(src + i), factor, load_f(at + i));
+    return;
+  }
   for (int i = threadIdx.x; i < H; i += blockDim.x) dst[i] = load_f(src + i) * factor;
 }
 
 // ------------------------------------------------------------------ gated activation
-// out = act(gate) * up, row = [gate (I) | up (I)] in 32-bit; act: 0 silu, 1 relu, 2 gelu by tanh
-// (0.5 z (1 + tanh(sqrt(2/pi) (z + 0.044715 z^3)))).  Computed in 32-bit, rounded once.
+// out = act(gate) * up, row = [gate (I) | up (I)] in 32-bit; act: ff_activation's numbers, or 4: the gate with limits
+// (clamped_gate).  Computed in 32-bit, rounded once.
 template <class TO>
 __global__ void __launch_bounds__(256)
     gated_act_kernel(const float* __restrict__ gu, int ld, const float* __restrict__ bias, const float* __restrict__ row_gate, int ldr,
-                     TO* __restrict__ out, int ldo, int I, int act) {
+                     TO* __restrict__ out, int ldo, int I, int act, float limit) {
   const int t = blockIdx.y;
   const int i = blockIdx.x * blockDim.x + threadIdx.x;
   if (i >= I) return;
@@ -456,12 +463,9 @@ __global__ void __launch_bounds__(256)
     g += bias[i];
     u += bias[I + i];
   }
-  if (row_gate) u *= 1.0f / (1.0f + expf(-row_gate[size_t(t) * ldr]));      // one gate logit per row
-  float a;
-  if (act == 1) a = fmaxf(g, 0.f);
-  else if (act == 2) a = 0.5f * g * (1.0f + tanhf(0.7978845608028654f * (g + 0.044715f * g * g * g)));
-  else a = g / (1.0f + expf(-g));
-  store_f(out + size_t(t) * ldo + i, a * u);
+  float v = act == 4 ? clamped_gate<float>(g, u, limit) : ff_activation(act, g) * u;
+  if (row_gate) v *= 1.0f / (1.0f + expf(-row_gate[size_t(t) * ldr]));      // one gate logit per row
+  store_f(out + size_t(t) * ldo + i, v);
 }
 
 // out[t, i] = act(in[t, i]) for feed-forwards without a gate: the same activations, computed in 32-bit, rounded once.
@@ -476,11 +480,7 @@ __global__ void __launch_bounds__(256)
   if (i >= I) return;
   float g = in[size_t(t) * ld + i];
   for (int sl = 1; sl < splits; ++sl) g += in[size_t(sl) * split_stride + size_t(t) * ld + i];
-  float a;
-  if (act == 1) a = fmaxf(g, 0.f);
-  else if (act == 2) a = 0.5f * g * (1.0f + tanhf(0.7978845608028654f * (g + 0.044715f * g * g * g)));
-  else a = g / (1.0f + expf(-g));
-  store_f(out + size_t(t) * ldo + i, a);
+  store_f(out + size_t(t) * ldo + i, ff_activation(act, g));
 }
 
 
@@ -493,23 +493,28 @@ extern "C" {
 const char* kvcm_hip_last_error() { return g_hip_error.c_str(); }
 
 int kvcm_embed_scaled(const int* ids, const void* table, int table_dtype, float* x, int T, int H, int V, float factor,
-                      hipStream_t s) {
+                      const int* positions, const void* pos_table, int P, hipStream_t s) {
   if (T == 0) return 0;
   KVCM_REQUIRE(T > 0 && H > 0 && V > 0, "embed_scaled: bad sizes T=%d H=%d V=%d", T, H, V);
-  if (table_dtype == kF32) embed_scaled_kernel<float><<<T, 256, 0, s>>>(ids, static_cast<const float*>(table), x, H, V, factor);
-  else if (table_dtype == kBF16) embed_scaled_kernel<bf16_t><<<T, 256, 0, s>>>(ids, static_cast<const bf16_t*>(table), x, H, V, factor);
+  KVCM_REQUIRE(!pos_table || (positions && P > 0), "embed_scaled: a table of position vectors needs the positions");
+  if (table_dtype == kF32)
+    embed_scaled_kernel<float><<<T, 256, 0, s>>>(ids, static_cast<const float*>(table), x, H, V, factor, positions, static_cast<const float*>(pos_table), P);
+  else if (table_dtype == kBF16)
+    embed_scaled_kernel<bf16_t><<<T, 256, 0, s>>>(ids, static_cast<const bf16_t*>(table), x, H, V, factor, positions, static_cast<const bf16_t*>(pos_table), P);
   else KVCM_REQUIRE(false, "embed_scaled: unknown table dtype %d", table_dtype);
   return launch_status("embed_scaled");
 }
 
-int kvcm_gated_act(const float* gate_up, int ld, const float* bias, const float* row_gate, int ldr, void* out, int out_dtype, int ldo, int T, int I, int act, hipStream_t s) {
+int kvcm_gated_act(const float* gate_up, int ld, const float* bias, const float* row_gate, int ldr, void* out, int out_dtype, int ldo, int T, int I, int act,
+                   float limit, hipStream_t s) {
   if (T == 0) return 0;
   KVCM_REQUIRE(T > 0 && I > 0 && ld >= 2 * I && ldo >= I, "gated_act: bad sizes T=%d I=%d", T, I);
   KVCM_REQUIRE(T <= 65535, "gated_act: too many rows for one launch (%d)", T);
-  KVCM_REQUIRE(act >= 0 && act <= 2, "gated_act: unknown activation %d (0 silu, 1 relu, 2 gelu_tanh)", act);
+  KVCM_REQUIRE(act >= 0 && act <= 4, "gated_act: unknown activation %d (0 silu, 1 relu, 2 gelu_tanh, 3 gelu, 4 clamped)", act);
+  KVCM_REQUIRE(act != 4 || limit > 0.f, "gated_act: a gate with limits needs a positive limit");
   const dim3 grid((I + 255) / 256, T);
-  if (out_dtype == kF32) gated_act_kernel<float><<<grid, 256, 0, s>>>(gate_up, ld, bias, row_gate, ldr, static_cast<float*>(out), ldo, I, act);
-  else if (out_dtype == kBF16) gated_act_kernel<bf16_t><<<grid, 256, 0, s>>>(gate_up, ld, bias, row_gate, ldr, static_cast<bf16_t*>(out), ldo, I, act);
+  if (out_dtype == kF32) gated_act_kernel<float><<<grid, 256, 0, s>>>(gate_up, ld, bias, row_gate, ldr, static_cast<float*>(out), ldo, I, act, limit);
+  else if (out_dtype == kBF16) gated_act_kernel<bf16_t><<<grid, 256, 0, s>>>(gate_up, ld, bias, row_gate, ldr, static_cast<bf16_t*>(out), ldo, I, act, limit);
   else KVCM_REQUIRE(false, "gated_act: unknown output dtype %d", out_dtype);
   return launch_status("gated_act");
 }
@@ -520,7 +525,7 @@ int kvcm_act_rows(const float* in, int ld, int splits, long long split_stride, v
   KVCM_REQUIRE(T > 0 && I > 0 && ld >= I && ldo >= I && in && out, "act_rows: bad sizes T=%d I=%d", T, I);
   KVCM_REQUIRE(splits >= 1 && split_stride >= 0, "act_rows: an input has at least one slice");
   KVCM_REQUIRE(T <= 65535, "act_rows: too many rows for one launch (%d)", T);
-  KVCM_REQUIRE(act >= 0 && act <= 2, "act_rows: unknown activation %d (0 silu, 1 relu, 2 gelu_tanh)", act);
+  KVCM_REQUIRE(act >= 0 && act <= 3, "act_rows: unknown activation %d (0 silu, 1 relu, 2 gelu_tanh, 3 gelu)", act);
   const dim3 grid((I + 255) / 256, T);
   const size_t stride = static_cast<size_t>(split_stride);
   if (out_dtype == kF32) act_rows_kernel<float><<<grid, 256, 0, s>>>(in, ld, splits, stride, static_cast<float*>(out), ldo, I, act);

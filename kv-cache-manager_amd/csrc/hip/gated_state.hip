@@ -5,6 +5,8 @@
 //       S <- g S;  u = beta (v - S^T k);  S <- S + k u^T;  o = S^T q
 //   delta 0 (state-space duality)     dt = softplus(a + dt_bias)
 //       S <- exp(-exp(a_log) dt) S + dt k v^T;  o = S^T q + d_skip v
+//   delta 0 with `decay` (a fixed decay per head)     q, k, v <- silu of what is given, where asked for
+//       S <- decay S + k v^T;  o = S^T q
 //
 // q and k come in `groups` heads of dk entries, v in `heads` heads of dv; head h reads group h / (heads / groups).  Everything
 // here is 32-bit.  A run that starts at position 0 starts from zero without reading its slot.
@@ -32,6 +34,8 @@ struct StateArgs {
   const float *q, *k, *v, *a, *b;      // 32-bit rows
   int ldq, ldk, ldv, lda, ldb;
   const float *dt_bias, *a_log, *d_skip;
+  const float* decay;                  // [heads]: a fixed decay (a, dt_bias, a_log, d_skip are not read)
+  int silu_in;
   float* o;
   int ldo;
   float* state;                        // [slots, heads, dk, dv]
@@ -90,8 +94,9 @@ __global__ void __launch_bounds__(256) gated_state_kernel(StateArgs A) {
       else if (pieces) S[c][il] = mine ? cst[size_t(i) * CW + j] : 0.f;
       else S[c][il] = (mine && !fresh) ? st[size_t(i) * dv + j] : 0.f;
     }
-  const float rate = -expf(A.a_log[head]), dtb = A.dt_bias[head];
-  const float skip = DELTA ? 0.f : A.d_skip[head];
+  const bool fixed = !DELTA && A.decay;
+  const float rate = fixed ? 0.f : -expf(A.a_log[head]), dtb = fixed ? 0.f : A.dt_bias[head];
+  const float skip = DELTA || fixed ? 0.f : A.d_skip[head], fixed_keep = fixed ? A.decay[head] : 0.f;
   const float q_scale = 1.0f / sqrtf(float(dk));
   float pf[PF], sa = 0.f, sb = 0.f;
   auto request = [&](int t0) {      // unconditional loads from clamped places, masked afterwards
@@ -111,19 +116,19 @@ __global__ void __launch_bounds__(256) gated_state_kernel(StateArgs A) {
     }
     const int t = threadIdx.x < TILE ? threadIdx.x : TILE - 1;
     const int row = t0 + t < r1 ? t0 + t : r1 - 1;
-    sa = A.a[size_t(row) * A.lda + head];
+    if (!fixed) sa = A.a[size_t(row) * A.lda + head];
     if constexpr (DELTA) sb = A.b[size_t(row) * A.ldb + head];
   };
   auto stage = [&]() {
 #pragma unroll
     for (int n = 0; n < PF; ++n) {
       const int e = threadIdx.x + n * 256;
-      if (e < TILE * V) tile[e / V][e % V] = pf[n];
+      if (e < TILE * V) tile[e / V][e % V] = !DELTA && A.silu_in ? silu<float>(pf[n]) : pf[n];      // (silu(0) = 0: what was masked stays 0)
     }
     if (threadIdx.x < TILE) {
       const float dt = softplus32(sa + dtb);
-      tile[threadIdx.x][V] = expf(rate * dt);
-      tile[threadIdx.x][V + 1] = DELTA ? 1.0f / (1.0f + expf(-sb)) : dt;
+      tile[threadIdx.x][V] = fixed ? fixed_keep : expf(rate * dt);
+      tile[threadIdx.x][V + 1] = DELTA ? 1.0f / (1.0f + expf(-sb)) : fixed ? 1.f : dt;
     }
     if constexpr (DELTA) {      // the lengths of the staged q and k: sixteen lanes a vector
       __syncthreads();
@@ -367,21 +372,23 @@ long long kvcm_gated_state_carry_floats(int rows, int S, int heads, int dk, int 
 }
 
 // q, k [T, groups*dk], v [T, heads*dv], a (and with delta b) [T, heads] at their own strides; dt_bias, a_log (and without delta
-// d_skip) [heads]; o [T, >= heads*dv]; state [slots, heads, dk, dv]; all 32-bit.  piece > 0: runs (max_run: the longest) are
+// d_skip) [heads]; decay [heads] (delta 0): a fixed decay in their place; silu_in (with decay): q, k and v are silu of what is
+// given; o [T, >= heads*dv]; state [slots, heads, dk, dv]; all 32-bit.  piece > 0: runs (max_run: the longest) are
 // walked in pieces of that many rows, with `carry` as scratch.
 int kvcm_gated_state(const float* q, int ldq, const float* k, int ldk, const float* v, int ldv, const float* a, int lda, const float* b,
-                     int ldb, const float* dt_bias, const float* a_log, const float* d_skip, int delta, float* o, int ldo, float* state,
+                     int ldb, const float* dt_bias, const float* a_log, const float* d_skip, const float* decay, int silu_in, int delta, float* o, int ldo, float* state,
                      const int* run_start, const int* seq_start, const int* state_slots, int S, int heads, int groups, int dk, int dv,
                      int T, int piece, int max_run, float* carry, long long carry_floats, hipStream_t s) {
   if (S == 0 || T == 0) return 0;
   KVCM_REQUIRE(S > 0 && T > 0 && heads > 0 && groups > 0 && dk > 0 && dv > 0, "gated_state: bad sizes S=%d heads=%d dk=%d dv=%d", S, heads, dk, dv);
   KVCM_REQUIRE(heads % groups == 0, "gated_state: %d heads are not a multiple of %d groups", heads, groups);
   KVCM_REQUIRE(dk <= 256, "gated_state: a key size of %d is not supported (up to 256)", dk);
-  KVCM_REQUIRE(ldq >= groups * dk && ldk >= groups * dk && ldv >= heads * dv && lda >= heads && (!delta || ldb >= heads) && ldo >= heads * dv,
+  KVCM_REQUIRE(ldq >= groups * dk && ldk >= groups * dk && ldv >= heads * dv && (decay || lda >= heads) && (!delta || ldb >= heads) && ldo >= heads * dv,
                "gated_state: row strides too small");
-  KVCM_REQUIRE(q && k && v && a && dt_bias && a_log && o && state && (delta ? b != nullptr : d_skip != nullptr), "gated_state: an operand is missing");
+  KVCM_REQUIRE(q && k && v && o && state && (decay || (a && dt_bias && a_log && (delta ? b != nullptr : d_skip != nullptr))), "gated_state: an operand is missing");
+  KVCM_REQUIRE(!(decay && delta) && (decay || !silu_in), "gated_state: a fixed decay beside the delta rule, or silu without one, is not supported");
   KVCM_REQUIRE(static_cast<long long>(heads) * ((dv + dk + 15) / 16) < (1ll << 31), "gated_state: too many heads");
-  StateArgs A = {q, k, v, a, b, ldq, ldk, ldv, lda, ldb, dt_bias, a_log, d_skip, o, ldo, state, run_start, seq_start, state_slots,
+  StateArgs A = {q, k, v, a, b, ldq, ldk, ldv, lda, ldb, dt_bias, a_log, d_skip, decay, silu_in, o, ldo, state, run_start, seq_start, state_slots,
                  heads, groups, dk, dv, 0, carry, piece, 1, 0};
   if (piece > 0) {
     KVCM_REQUIRE(max_run > 0 && carry && carry_floats >= kvcm_gated_state_carry_floats(T, S, heads, dk, dv, delta, piece),

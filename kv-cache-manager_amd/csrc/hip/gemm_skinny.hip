@@ -38,7 +38,7 @@ union Frag {
 template <int MT, class TO, bool SWIGLU>
 __global__ void __launch_bounds__(256)
     gemm_skinny_kernel(const uint16_t* __restrict__ X, const uint16_t* __restrict__ W, float* __restrict__ partials,
-                       TO* __restrict__ out, int M, int N, int K, int ldx, int ldw, int ldo, int S) {
+                       TO* __restrict__ out, int M, int N, int K, int ldx, int ldw, int ldo, int S, float limit) {
   __shared__ f32x4 red[4][MT][kWave];
   const int wave = threadIdx.x / kWave, lane = threadIdx.x % kWave;
   const int r = lane % 16, kq = lane / 16;
@@ -140,9 +140,14 @@ __global__ void __launch_bounds__(256)
       for (int i = 0; i < 4; ++i) {
         const int m = t * 16 + (l / 16) * 4 + i;
         if (m >= M) continue;
+        TO* dst = out + size_t(m) * ldo + n0 + l % 16;
+        if (limit > 0.f) {
+          store_f(dst, clamped_gate<TO>(g[i], up[i], limit));
+          continue;
+        }
         const float x = round_to<TO>(g[i]);
         const float act = silu<TO>(x);
-        store_f(out + size_t(m) * ldo + n0 + l % 16, round_to<TO>(act) * round_to<TO>(up[i]));
+        store_f(dst, round_to<TO>(act) * round_to<TO>(up[i]));
       }
     }
     return;
@@ -176,7 +181,8 @@ __global__ void __launch_bounds__(256)
 // wave streams its own 16 weight rows from HBM and multiplies them with the staged rows.  No reduction
 // between waves; split-K partial sums as above.  More than 128 rows run as row blocks of 128
 // (blockIdx.z), each streaming the weights again.
-// SWIGLU: a wave's tile is 8 gate + 8 up rows, it stores 8 activation columns.
+// SWIGLU: a wave's tile is 8 gate + 8 up rows, it stores 8 activation columns (limit > 0: of the gate with limits, whose
+// gate and up values are not rounded on the way).
 constexpr int kXPad = 8;    // bfloat16 of padding per staged row, so that rows spread over the banks
 constexpr int kRowBlock = 128;
 
@@ -184,7 +190,7 @@ template <int MT, int DEPTH, class TO, bool SWIGLU, int NWV>
 __global__ void __launch_bounds__(NWV * kWave)
     gemm_rows_kernel(const uint16_t* __restrict__ X, const uint16_t* __restrict__ W, float* __restrict__ partials,
                      TO* __restrict__ out, int M, int N, int K, int ldx, int ldw, int ldo, int S,
-                     const float* __restrict__ ss_in, int tiles_in, float eps) {
+                     const float* __restrict__ ss_in, int tiles_in, float eps, float limit) {
   constexpr int kPassRows = NWV * kWave / 4;                      // rows the workgroup's threads stage at a time (x 64 k)
   constexpr int RP = (MT * 16 + kPassRows - 1) / kPassRows;       // staging passes
   __shared__ __attribute__((aligned(16))) uint16_t xs[2][MT * 16][DEPTH * kUnit + kXPad];
@@ -332,9 +338,14 @@ __global__ void __launch_bounds__(NWV * kWave)
       for (int i = 0; i < 4; ++i) {
         const int m = row_base + t * 16 + kq * 4 + i;
         if (m >= M) continue;
+        TO* dst = out + size_t(m) * ldo + c0 + r;
+        if (limit > 0.f) {
+          store_f(dst, clamped_gate<TO>(acc[t][i], up[i], limit));
+          continue;
+        }
         const float x = round_to<TO>(acc[t][i]);
         const float act = silu<TO>(x);
-        store_f(out + size_t(m) * ldo + c0 + r, round_to<TO>(act) * round_to<TO>(up[i]));
+        store_f(dst, round_to<TO>(act) * round_to<TO>(up[i]));
       }
     }
     return;
@@ -413,13 +424,13 @@ static int rows_splits(int M, int N, int K) {
 // several), two k-depths: four units per trip up to 64 rows, two beyond (LDS holds rows x depth).
 template <class TO, bool SWIGLU, int NWV>
 static void launch_rows_n(hipStream_t st, const uint16_t* x, const uint16_t* w, float* partials, TO* out, int M, int N,
-                          int K, int ldx, int ldw, int ldo, int S, const float* ss_in, int tiles_in, float eps) {
+                          int K, int ldx, int ldw, int ldo, int S, const float* ss_in, int tiles_in, float eps, float limit) {
   const int mt = rows_tiles_m(M);
   const int tiles = N / (SWIGLU ? 8 : 16);
   const dim3 grid((tiles + NWV - 1) / NWV, S, row_blocks(M));
 #define KVCM_ROWS(MT, DEPTH) \
   gemm_rows_kernel<MT, DEPTH, TO, SWIGLU, NWV><<<grid, NWV * kWave, 0, st>>>(x, w, partials, out, M, N, K, ldx, ldw, ldo, S, \
-                                                                             ss_in, tiles_in, eps)
+                                                                             ss_in, tiles_in, eps, limit)
   switch (mt) {
     case 1: KVCM_ROWS(1, 4); break;
     case 2: KVCM_ROWS(2, 4); break;
@@ -435,10 +446,10 @@ static void launch_rows_n(hipStream_t st, const uint16_t* x, const uint16_t* w, 
 // tiles) keeps four waves.
 template <class TO, bool SWIGLU>
 static void launch_rows(hipStream_t st, const uint16_t* x, const uint16_t* w, float* partials, TO* out, int M, int N, int K,
-                        int ldx, int ldw, int ldo, int S, const float* ss_in = nullptr, int tiles_in = 0, float eps = 0.f) {
+                        int ldx, int ldw, int ldo, int S, const float* ss_in = nullptr, int tiles_in = 0, float eps = 0.f, float limit = 0.f) {
   const long long units = static_cast<long long>(N / (SWIGLU ? 8 : 16)) * row_blocks(M) * S;
   const int waves = sizeof(TO) == 4 || (S == 1 && !SWIGLU) ? 4 : rows_waves(units, rows_tiles_m(M));
-#define KVCM_WAVES(NWV) launch_rows_n<TO, SWIGLU, NWV>(st, x, w, partials, out, M, N, K, ldx, ldw, ldo, S, ss_in, tiles_in, eps)
+#define KVCM_WAVES(NWV) launch_rows_n<TO, SWIGLU, NWV>(st, x, w, partials, out, M, N, K, ldx, ldw, ldo, S, ss_in, tiles_in, eps, limit)
   if constexpr (sizeof(TO) == 4) {
     KVCM_WAVES(4);
   } else {
@@ -501,7 +512,7 @@ int kvcm_gemm_skinny(const void* X, const void* W, float* partials, void* out, i
   }
   const dim3 grid(N / 16, S);
 #define KVCM_SKINNY(MT, TO) \
-  gemm_skinny_kernel<MT, TO, false><<<grid, 256, 0, st>>>(x, w, partials, static_cast<TO*>(out), M, N, K, ldx, ldw, ldo, S)
+  gemm_skinny_kernel<MT, TO, false><<<grid, 256, 0, st>>>(x, w, partials, static_cast<TO*>(out), M, N, K, ldx, ldw, ldo, S, 0.f)
   if (out_dtype == kBF16) {
     if (mt == 1) KVCM_SKINNY(1, bf16_t); else if (mt == 2) KVCM_SKINNY(2, bf16_t); else if (mt == 3) KVCM_SKINNY(3, bf16_t); else KVCM_SKINNY(4, bf16_t);
   } else {
@@ -521,9 +532,9 @@ int kvcm_gemm_skinny_swiglu_supported(int M, int I, int K) {
   return M <= 64 && I / 8 >= 320;
 }
 
-// W [2 I, K] (gate rows, then up rows); out [M, I].
+// W [2 I, K] (gate rows, then up rows); out [M, I].  limit > 0: the gate with limits (clamped_gate) instead of silu(gate) * up.
 int kvcm_gemm_skinny_swiglu(const void* X, const void* W, void* out, int out_dtype, int M, int I, int K, int ldx,
-                            int ldw, int ldo, hipStream_t st) {
+                            int ldw, int ldo, float limit, hipStream_t st) {
   KVCM_REQUIRE(kvcm_gemm_skinny_swiglu_supported(M, I, K), "gemm_skinny_swiglu: unsupported shape M=%d I=%d K=%d", M, I, K);
   KVCM_REQUIRE(ldx % 8 == 0 && ldw % 8 == 0 && reinterpret_cast<uintptr_t>(X) % 16 == 0 &&
                    reinterpret_cast<uintptr_t>(W) % 16 == 0,
@@ -534,13 +545,13 @@ int kvcm_gemm_skinny_swiglu(const void* X, const void* W, void* out, int out_dty
   const uint16_t* w = static_cast<const uint16_t*>(W);
   const int mt = (M + 15) / 16;
   if (swiglu_shares_rows(M, I)) {
-    if (out_dtype == kBF16) launch_rows<bf16_t, true>(st, x, w, nullptr, static_cast<bf16_t*>(out), M, I, K, ldx, ldw, ldo, 1);
-    else launch_rows<float, true>(st, x, w, nullptr, static_cast<float*>(out), M, I, K, ldx, ldw, ldo, 1);
+    if (out_dtype == kBF16) launch_rows<bf16_t, true>(st, x, w, nullptr, static_cast<bf16_t*>(out), M, I, K, ldx, ldw, ldo, 1, nullptr, 0, 0.f, limit);
+    else launch_rows<float, true>(st, x, w, nullptr, static_cast<float*>(out), M, I, K, ldx, ldw, ldo, 1, nullptr, 0, 0.f, limit);
     return launch_status("gemm_rows_swiglu");
   }
   const dim3 grid(I / 8, 1);
 #define KVCM_SKINNY(MT, TO) \
-  gemm_skinny_kernel<MT, TO, true><<<grid, 256, 0, st>>>(x, w, nullptr, static_cast<TO*>(out), M, I, K, ldx, ldw, ldo, 1)
+  gemm_skinny_kernel<MT, TO, true><<<grid, 256, 0, st>>>(x, w, nullptr, static_cast<TO*>(out), M, I, K, ldx, ldw, ldo, 1, limit)
   if (out_dtype == kBF16) {
     if (mt == 1) KVCM_SKINNY(1, bf16_t); else if (mt == 2) KVCM_SKINNY(2, bf16_t); else if (mt == 3) KVCM_SKINNY(3, bf16_t); else KVCM_SKINNY(4, bf16_t);
   } else {

@@ -68,7 +68,7 @@ int kvcm_add_residual(float* x, const void* y, int dtype, long long n, hipStream
 // ---- products --------------------------------------------------------------------------------
 int kvcm_gemm_skinny_swiglu_supported(int M, int I, int K);
 int kvcm_gemm_skinny_swiglu(const void* X, const void* W, void* out, int out_dtype, int M, int I, int K, int ldx,
-                            int ldw, int ldo, hipStream_t stream);
+                            int ldw, int ldo, float limit, hipStream_t stream);
 int kvcm_gemm_f32(const float* X, const float* W, float* Y, int M, int N, int K, int ldx, int ldw, int ldy, hipStream_t s);
 int kvcm_gemm_bf16(const void* X, const void* W, void* Y, int out_dtype, int M, int N, int K, int ldx, int ldw, int ldy,
                    hipStream_t s);
@@ -148,8 +148,9 @@ int kvcm_probe_phases(const void* weights, const long long* phase_bytes, int pha
 // ---- parts of sequence models beyond the dense decoder ----------------------------------------------
 // (elementwise.hip) the embedding times a factor; act(gate) * up with act 0 silu, 1 relu, 2 gelu by tanh
 int kvcm_embed_scaled(const int* ids, const void* table, int table_dtype, float* x, int T, int H, int V, float factor,
-                      hipStream_t s);
-int kvcm_gated_act(const float* gate_up, int ld, const float* bias, const float* row_gate, int ldr, void* out, int out_dtype, int ldo, int T, int I, int act, hipStream_t s);
+                      const int* positions, const void* pos_table, int P, hipStream_t s);
+int kvcm_gated_act(const float* gate_up, int ld, const float* bias, const float* row_gate, int ldr, void* out, int out_dtype, int ldo, int T, int I, int act,
+                   float limit, hipStream_t s);
 // (norm_chain.hip) 32-bit RMS norms chained along a row: two branches combined, normed, added to the stream, the
 // stream normed again; the norm of every head with a weight and a sigmoid gate
 int kvcm_rmsnorm_chain(float* x, const float* a, int a_splits, const float* b, int b_splits, long long split_stride,
@@ -179,7 +180,7 @@ int kvcm_attention_window_pool(const void* q, int dtype, int ldq, void* out, int
                                const float* pk, const float* pv, const int* tables, int table_stride, const int* row_seq,
                                const int* ctx_lens, const float* head_scale, const float* dist_slope, const float* gate, int ldg,
                                int T, int nh, int nkv, int d, int dv, int B, float scale, int window, int P, int E, int keep_first,
-                               float softcap, int chunk, int sink, float out_scale, hipStream_t s);
+                               float softcap, int chunk, int sink, const float* sink_logit, int gate_heads, float out_scale, hipStream_t s);
 // as rotate_store, after q and k were divided by the root mean square of their whole stretch (times a weight) and v was
 // blended with another layer's values of the same row
 int kvcm_norm_rotate_store(const float* src, int ld, const float* wq, const float* wk, float eps, const float* v_other, int ldvo,
@@ -192,7 +193,7 @@ int kvcm_attention_window_pool_tiles(const void* q, int ldq, void* out, int ldo,
                                      const float* pk, const float* pv, const int* tables, int table_stride,
                                      const int* run_start, const int* seq_start, const float* head_scale, const float* dist_slope,
                                      const float* gate, int ldg, int S, int max_run, int nh, int nkv, int d, int dv, int B, float scale, int window, int P,
-                                     int E, int keep_first, float softcap, int chunk, int sink, float out_scale, hipStream_t s);
+                                     int E, int keep_first, float softcap, int chunk, int sink, const float* sink_logit, int gate_heads, float out_scale, hipStream_t s);
 // (selective_scan.hip, delta_rule.hip) recurrences with a 32-bit state per sequence
 int kvcm_selective_scan(const void* x, int dtype, int ldx, const float* dt_lin, int lddt, const float* dt_bias,
                         const float* bc, int ldbc, int off_b, int off_c, const float* a_log, const float* dskip,
@@ -238,11 +239,12 @@ int kvcm_stream_terms(float* x, const float* a, int a_splits, float a_factor, co
                       const float* c, int c_splits, float c_factor, long long split_stride, const float* bias, const float* again,
                       const int* rows, const float* w, void* out, int out_dtype, int R, int H, float eps, hipStream_t s);
 int kvcm_group_norm_gate(const float* y, int ldy, const float* z, int ldz, const float* w, void* out, int out_dtype, int ldo, int T,
-                         int groups, int size, float eps, hipStream_t s);
-// (gated_state.hip) the gated delta rule (delta 1) and the state-space recurrence with one decay per head (delta 0)
+                         int groups, int size, float eps, int after, hipStream_t s);
+// (gated_state.hip) the gated delta rule (delta 1), the state-space recurrence with one decay per head (delta 0), and a state
+// with a fixed decay (delta 0, decay)
 long long kvcm_gated_state_carry_floats(int rows, int S, int heads, int dk, int dv, int delta, int piece);
 int kvcm_gated_state(const float* q, int ldq, const float* k, int ldk, const float* v, int ldv, const float* a, int lda, const float* b,
-                     int ldb, const float* dt_bias, const float* a_log, const float* d_skip, int delta, float* o, int ldo, float* state,
+                     int ldb, const float* dt_bias, const float* a_log, const float* d_skip, const float* decay, int silu_in, int delta, float* o, int ldo, float* state,
                      const int* run_start, const int* seq_start, const int* state_slots, int S, int heads, int groups, int dk, int dv,
                      int T, int piece, int max_run, float* carry, long long carry_floats, hipStream_t s);
 // (mlstm.hip) a matrix memory with exponential gates, walked token by token
@@ -252,12 +254,12 @@ int kvcm_mlstm_scan(const float* q, int ldq, const float* k, int ldk, const floa
                     const int* seq_start, const int* state_slots, int S, int heads, int dk, int dv, int T, int max_run,
                     hipStream_t s);
 // (moe.hip) a routed feed-forward: the choice of experts, and the experts' two products a row at a time
-int kvcm_moe_route(const float* logits, int ld, int splits, long long split_stride, int E, int top, int over_chosen, float factor, int* chosen,
+int kvcm_moe_route(const float* logits, int ld, int splits, long long split_stride, int E, int top, int mode, float factor, int* chosen,
                    float* weight, int T, hipStream_t s);
 int kvcm_moe_table_route(const int* tokens, const int* table, int vocab, int ld, int top, int* chosen, float* weight, int T,
                          hipStream_t s);
 int kvcm_moe_up(const void* h, int dtype, int ldh, const void* w_up, const int* chosen, void* act, int T, int K, int F, int top,
-                int E, int gated, hipStream_t s);
+                int E, int kind, const float* in_weight, hipStream_t s);
 int kvcm_moe_down(const void* act, int dtype, const void* w_down, const int* chosen, const float* weight, const float* add,
                   float* out, int T, int F, int H, int top, int E, hipStream_t s);
 // (moe_grouped.hip) the routed feed-forward for many rows: pairs grouped by expert, tiles on the matrix cores
@@ -265,7 +267,7 @@ int kvcm_moe_grouped_supported(int K, int F, int E);
 int kvcm_moe_grouped_max_tiles(int n, int E);
 int kvcm_moe_grouped(const void* h, int ldh, const void* w_up, const void* w_down, const int* chosen, const float* weight,
                      int* order, int* tiles, void* act, float* y, const float* add, float* out, int T, int K, int F, int H,
-                     int top, int E, int gated, hipStream_t s);
+                     int top, int E, int kind, int weigh_input, hipStream_t s);
 
 // ---- recorded steps ---------------------------------------------------------------------------
 // A step program is the list of launches of one step, recorded once for a step shape and replayed

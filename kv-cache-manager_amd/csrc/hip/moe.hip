@@ -1,14 +1,18 @@
-// A routed feed-forward: every row picks `top` of E small experts by the softmax of its router logits and gets the
-// sum of their outputs weighted by the chosen scores as they are (not renormalized).
+// A routed feed-forward: every row picks `top` of E small experts by the scores of its router logits (softmax or sigmoid) and
+// gets the sum of their outputs weighted by the chosen scores as they are (not renormalized); or the scores weigh what goes
+// into the experts instead of what comes out.
 //
 //   moe_route      32-bit router logits [T, E] -> chosen[T, top] (expert numbers, best first; equal scores: the lower
-//                  number) and weight[T, top]: their softmax scores over all E, or (over_chosen) the softmax over the
-//                  chosen logits alone, which add up to one; times a constant factor.  One wave per row.
+//                  number) and weight[T, top]: their softmax scores over all E (mode 0), the softmax over the chosen
+//                  logits alone, which add up to one (mode 1), or sigmoid of each chosen logit on its own (mode 2, which
+//                  chooses the same experts: sigmoid grows with the logit); times a constant factor.  One wave per row.
 //   moe_table_route  chosen[T, top] = table[token of the row, :] (a table of expert numbers per token id), weight = 1 / top
-//   moe_up         act[T, top, F] = a(W_up[e] h) for each row's chosen experts, a = square of relu, rounded to the
-//                  compute dtype; or, gated, act = silu(W_gate[e] h) * (W_up[e] h) with the two matrices of an expert
-//                  stored as one, their rows interleaved sixteen at a time (gate 0..15, up 0..15, gate 16..31, ...)
-//   moe_down       out[T, H] (32-bit) = (add +) sum over the row's slots of weight * W_down[e] act[slot]
+//   moe_up         act[T, top, F] = a(W_up[e] h) for each row's chosen experts, a = square of relu (act 0) or gelu by the
+//                  error function (act 2), rounded to the compute dtype; or, gated (act 1), silu(W_gate[e] h) * (W_up[e] h)
+//                  with the two matrices of an expert stored as one, their rows interleaved sixteen at a time (gate 0..15,
+//                  up 0..15, gate 16..31, ...).  in_weight[T, top]: the expert reads in_weight * h (the factor is applied to
+//                  the 32-bit sums, which are linear in h)
+//   moe_down       out[T, H] (32-bit) = (add +) sum over the row's slots of weight * W_down[e] act[slot] (no weight: 1)
 //
 // The two products here take a row at a time: a workgroup owns one (row, slot) and a stretch of output columns, keeps
 // the row in LDS as 32-bit values and streams the chosen expert's weight rows, a wave per output column, 16 bytes per
@@ -26,7 +30,7 @@ constexpr int kMoeMaxTop = 16;
 constexpr int kMoeMaxExperts = 1024;      // a row's logits are kept in LDS while its experts are picked
 
 __global__ void __launch_bounds__(256)
-    moe_route_kernel(const float* __restrict__ logits, int ld, int splits, size_t split_stride, int E, int top, int over_chosen,
+    moe_route_kernel(const float* __restrict__ logits, int ld, int splits, size_t split_stride, int E, int top, int mode,
                      float factor, int* __restrict__ chosen, float* __restrict__ weight, int T) {
   // up to 64 experts a lane group: the row's logits are formed once (a router product that was split along K arrives as
   // slices, which are added here in their order) and kept in LDS
@@ -65,13 +69,13 @@ __global__ void __launch_bounds__(256)
       if (ob > best || (ob == best && oa < at)) { best = ob; at = oa; }
     }
     taken[s] = at;
-    picked[s] = expf(best - mx);      // the first pick is the largest logit: exp(0)
+    picked[s] = mode == 2 ? 1.0f / (1.0f + expf(-best)) : expf(best - mx);      // (the first pick is the largest logit: exp(0))
     if (lane == 0) {
       chosen[size_t(row) * top + s] = at;
-      if (!over_chosen) weight[size_t(row) * top + s] = picked[s] * inv * factor;
+      if (mode != 1) weight[size_t(row) * top + s] = picked[s] * (mode == 2 ? 1.0f : inv) * factor;
     }
   }
-  if (over_chosen && lane == 0) {
+  if (mode == 1 && lane == 0) {
     float among = 0.f;
     for (int s = 0; s < top; ++s) among += picked[s];
     const float inv_among = factor / among;
@@ -154,7 +158,7 @@ __device__ __forceinline__ void wave_dots(const float* xs, const T* w, size_t st
 template <class T, int CW>
 __global__ void __launch_bounds__(256)
     moe_up_kernel(const T* __restrict__ h, int ldh, const T* __restrict__ w_up, const int* __restrict__ chosen,
-                  T* __restrict__ act, int K, int F, int top, int E, int gated) {
+                  T* __restrict__ act, int K, int F, int top, int E, int kind, const float* __restrict__ in_weight) {
   extern __shared__ __attribute__((aligned(16))) float xs[];
   const int item = blockIdx.x, row = item / top;
   const int e = chosen[item];
@@ -167,21 +171,22 @@ __global__ void __launch_bounds__(256)
   if (c0 >= F) return;
   const int cols = F - c0 < CW ? F - c0 : CW;
   float z[CW];
-  if (gated) {
+  const float g = in_weight ? in_weight[item] : 1.f;
+  if (kind == 1) {
     // (F is a multiple of 16 and c0 one of CW <= 4: the wave's columns lie in one stretch of sixteen)
     const T* gate = w_up + (size_t(e) * 2 * F + size_t(c0 / 16) * 32 + c0 % 16) * K;
     float u[CW];
     wave_dots<T, CW>(xs, gate, K, cols, K, lane, vec, z);
     wave_dots<T, CW>(xs, gate + size_t(16) * K, K, cols, K, lane, vec, u);
     if (lane == 0)
-      for (int c = 0; c < cols; ++c) store_f(act + size_t(item) * F + c0 + c, silu<T>(z[c]) * u[c]);
+      for (int c = 0; c < cols; ++c) store_f(act + size_t(item) * F + c0 + c, silu<T>(g * z[c]) * (g * u[c]));
     return;
   }
   wave_dots<T, CW>(xs, w_up + (size_t(e) * F + c0) * K, K, cols, K, lane, vec, z);
   if (lane == 0)
     for (int c = 0; c < cols; ++c) {
-      const float r = fmaxf(z[c], 0.f);
-      store_f(act + size_t(item) * F + c0 + c, r * r);
+      const float y = g * z[c], r = fmaxf(y, 0.f);
+      store_f(act + size_t(item) * F + c0 + c, kind == 2 ? ff_activation(3, y) : r * r);
     }
 }
 
@@ -209,7 +214,7 @@ __global__ void __launch_bounds__(256)
     if (e < 0 || e >= E) continue;
     float z[CW];
     wave_dots<T, CW>(xs + s * F4, w_down + (size_t(e) * H + c0) * F, F, cols, F, lane, vec, z);
-    const float g = weight[size_t(row) * top + s];
+    const float g = weight ? weight[size_t(row) * top + s] : 1.f;
 #pragma unroll
     for (int c = 0; c < CW; ++c) acc[c] = fmaf(g, z[c], acc[c]);
   }
@@ -230,14 +235,15 @@ using namespace kvcm;
 
 extern "C" {
 
-int kvcm_moe_route(const float* logits, int ld, int splits, long long split_stride, int E, int top, int over_chosen, float factor, int* chosen,
+int kvcm_moe_route(const float* logits, int ld, int splits, long long split_stride, int E, int top, int mode, float factor, int* chosen,
                    float* weight, int T, hipStream_t s) {
   if (T == 0) return 0;
   KVCM_REQUIRE(T > 0 && E > 0 && top > 0 && top <= E && ld >= E, "moe_route: bad sizes T=%d experts=%d top=%d", T, E, top);
   KVCM_REQUIRE(top <= kMoeMaxTop, "moe_route: %d experts a row are not supported (up to %d)", top, kMoeMaxTop);
   KVCM_REQUIRE(E <= kMoeMaxExperts, "moe_route: %d experts are not supported (up to %d)", E, kMoeMaxExperts);
+  KVCM_REQUIRE(mode >= 0 && mode <= 2, "moe_route: unknown kind of weights %d (0 softmax, 1 softmax over the chosen, 2 sigmoid)", mode);
   KVCM_REQUIRE(splits >= 1 && split_stride >= 0, "moe_route: the logits have at least one slice");
-  moe_route_kernel<<<(T + 3) / 4, 256, 0, s>>>(logits, ld, splits, static_cast<size_t>(split_stride), E, top, over_chosen, factor, chosen, weight, T);
+  moe_route_kernel<<<(T + 3) / 4, 256, 0, s>>>(logits, ld, splits, static_cast<size_t>(split_stride), E, top, mode, factor, chosen, weight, T);
   return launch_status("moe_route");
 }
 
@@ -252,13 +258,15 @@ int kvcm_moe_table_route(const int* tokens, const int* table, int vocab, int ld,
   return launch_status("moe_table_route");
 }
 
-// h [T, K] and act [T * top, F] in dtype; w_up [E, F, K] contiguous: act = square(relu(W_up[chosen] h)).  gated: w_up
-// [E, 2F, K], an expert's gate and up rows interleaved sixteen at a time: act = silu(W_gate[chosen] h) * (W_up[chosen] h).
+// h [T, K] and act [T * top, F] in dtype; w_up [E, F, K] contiguous: act = square(relu(W_up[chosen] h)) (kind 0) or
+// gelu(W_up[chosen] h) (kind 2).  kind 1, gated: w_up [E, 2F, K], an expert's gate and up rows interleaved sixteen at a time:
+// act = silu(W_gate[chosen] h) * (W_up[chosen] h).  in_weight [T * top] or null: a factor on what the expert reads.
 int kvcm_moe_up(const void* h, int dtype, int ldh, const void* w_up, const int* chosen, void* act, int T, int K, int F, int top,
-                int E, int gated, hipStream_t s) {
+                int E, int kind, const float* in_weight, hipStream_t s) {
   if (T == 0) return 0;
   KVCM_REQUIRE(T > 0 && K > 0 && F > 0 && top > 0 && E > 0 && ldh >= K, "moe_up: bad sizes");
-  KVCM_REQUIRE(!gated || F % 16 == 0, "moe_up: gated experts of %d columns are not supported (a multiple of 16)", F);
+  KVCM_REQUIRE(kind >= 0 && kind <= 2, "moe_up: unknown kind of experts %d (0 relu2, 1 silu gated, 2 gelu)", kind);
+  KVCM_REQUIRE(kind != 1 || F % 16 == 0, "moe_up: gated experts of %d columns are not supported (a multiple of 16)", F);
   KVCM_REQUIRE(static_cast<long long>(T) * top < (1ll << 31) && (F + 3) / 4 <= 65535, "moe_up: too many rows or columns");
   KVCM_REQUIRE(K * sizeof(float) <= 64 * 1024, "moe_up: rows of %d values do not fit the local memory", K);
   KVCM_REQUIRE(reinterpret_cast<uintptr_t>(w_up) % 16 == 0, "moe_up: weights must be 16-byte aligned");
@@ -268,7 +276,7 @@ int kvcm_moe_up(const void* h, int dtype, int ldh, const void* w_up, const int* 
   const size_t lds = K * sizeof(float);
 #define KVCM_MOE_UP(TT, CW)                                                                                              \
   moe_up_kernel<TT, CW><<<grid, 256, lds, s>>>(static_cast<const TT*>(h), ldh, static_cast<const TT*>(w_up), chosen,     \
-                                               static_cast<TT*>(act), K, F, top, E, gated)
+                                               static_cast<TT*>(act), K, F, top, E, kind, in_weight)
   if (dtype == kF32) { if (cw == 4) KVCM_MOE_UP(float, 4); else if (cw == 2) KVCM_MOE_UP(float, 2); else KVCM_MOE_UP(float, 1); }
   else { if (cw == 4) KVCM_MOE_UP(bf16_t, 4); else if (cw == 2) KVCM_MOE_UP(bf16_t, 2); else KVCM_MOE_UP(bf16_t, 1); }
 #undef KVCM_MOE_UP

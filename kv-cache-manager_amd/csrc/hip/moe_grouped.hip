@@ -7,11 +7,13 @@
 //                  the number of tiles in front.  One workgroup; places inside a group are handed out by an atomic
 //                  counter in LDS, so the order inside a group may differ from run to run, which changes no result: a
 //                  pair's row of a tile is computed from that row alone.
-//   moe_grouped    UP:   act[place, :] = square(relu(W_up[e] h[row of the pair]))           (bfloat16, in grouped order)
+//   moe_grouped    UP:   act[place, :] = square(relu(W_up[e] h[row of the pair])), or gelu of it (bfloat16, in grouped order)
 //                  GATED UP: act[place, :] = silu(W_gate[e] h) * (W_up[e] h); the two matrices of an expert are stored as
 //                        one of 2F rows, interleaved sixteen at a time (gate 0..15, up 0..15, gate 16..31, ...), so that a
 //                        lane's neighbouring 16 x 16 tiles hold the gate and the up value of one column
 //                  DOWN: y[pair, :]   = weight[pair] * W_down[e] act[place, :]               (32-bit, by pair)
+//                  The pairs' weights may act on the other side instead: UP then reads weight * h (the factor is applied to
+//                  its 32-bit sums) and DOWN weighs nothing.
 //                  Tile 128 pairs x 128 columns per workgroup of four waves (64 x 64 each: 4 x 4 matrix instructions of
 //                  16 x 16 x 32), K advanced 64 at a time through LDS, the next 64 on their way in registers meanwhile.
 //   moe_combine    out[row, :] = (add[row, :] +) sum over the row's slots, in slot order, of y[row * top + slot, :]
@@ -59,7 +61,7 @@ __global__ void __launch_bounds__(1024)
   }
 }
 
-enum : int { kDown = 0, kUp = 1, kUpGated = 2 };
+enum : int { kDown = 0, kUp = 1, kUpGated = 2, kUpGelu = 3 };
 
 // N: rows of an expert's matrix (2F for the gated form); the output has N columns (F for the gated form)
 template <int MODE>
@@ -165,7 +167,7 @@ __global__ void __launch_bounds__(256)
         const int c = n0 + wn * 64 + c4;
         if (m >= rows || c >= N) continue;
         const int pair = pair_of[m];
-        const float g = weight[pair];
+        const float g = weight ? weight[pair] : 1.f;
         const float4 v = *reinterpret_cast<const float4*>(mine + rl * kPitch + c4);
         float* dst = static_cast<float*>(out) + static_cast<long long>(pair) * N + c;
         if (c + 3 < N && N % 4 == 0) {
@@ -186,7 +188,7 @@ __global__ void __launch_bounds__(256)
       const int m = wm * 64 + i * 16 + (lane / 16) * 4 + r;
       if (m >= rows) continue;
       const int pair = pair_of[m];
-      const float g = MODE != kDown ? 1.f : weight[pair];
+      const float g = weight ? weight[pair] : 1.f;      // (the down form returned above: here a factor on what the expert reads)
       if constexpr (MODE == kUpGated) {
 #pragma unroll
         for (int j = 0; j < 4; j += 2) {      // tile j: sixteen gate columns, tile j + 1: the same sixteen up columns
@@ -194,20 +196,16 @@ __global__ void __launch_bounds__(256)
           if (c >= N) continue;
           const int col = (n0 + wn * 64 + j * 16) / 2 + lane % 16;
           static_cast<uint16_t*>(out)[static_cast<long long>(p0 + m) * (N / 2) + col] =
-              float_to_bf16_bits(silu<bf16_t>(acc[i][j][r]) * acc[i][j + 1][r]);
+              float_to_bf16_bits(silu<bf16_t>(g * acc[i][j][r]) * (g * acc[i][j + 1][r]));
         }
       } else {
 #pragma unroll
         for (int j = 0; j < 4; ++j) {
           const int c = n0 + wn * 64 + j * 16 + lane % 16;
           if (c >= N) continue;
-          const float v = acc[i][j][r];
-          if (MODE == kUp) {
-            const float z = fmaxf(v, 0.f);
-            static_cast<uint16_t*>(out)[static_cast<long long>(p0 + m) * N + c] = float_to_bf16_bits(z * z);
-          } else {
-            static_cast<float*>(out)[static_cast<long long>(pair) * N + c] = g * v;
-          }
+          const float v = g * acc[i][j][r], z = fmaxf(v, 0.f);
+          static_cast<uint16_t*>(out)[static_cast<long long>(p0 + m) * N + c] =
+              float_to_bf16_bits(MODE == kUpGelu ? ff_activation(3, v) : z * z);
         }
       }
     }
@@ -239,11 +237,12 @@ int kvcm_moe_grouped_max_tiles(int n, int E) { return (n + kGM - 1) / kGM + E; }
 
 // h [T, K] bfloat16; w_up [E, F, K], w_down [E, H, F] bfloat16; chosen [T * top], weight [T * top]; work memory:
 // order [T * top] and tiles [3 * max_tiles + 1] (int32), act [T * top, F] (bfloat16), y [T * top, H] (32-bit); out [T, H] 32-bit.
-// gated: w_up [E, 2F, K] (gate and up rows interleaved sixteen at a time), act = silu(gate) * up.  add [T, H] 32-bit or
-// null: out = add + the experts' sum.
+// kind 0: act = square(relu(up)); 2: gelu(up); 1, gated: w_up [E, 2F, K] (gate and up rows interleaved sixteen at a time), act =
+// silu(gate) * up.  weigh_input: the weights are factors on what the experts read, not on what they give.  add [T, H] 32-bit
+// or null: out = add + the experts' sum.
 int kvcm_moe_grouped(const void* h, int ldh, const void* w_up, const void* w_down, const int* chosen, const float* weight,
                      int* order, int* tiles, void* act, float* y, const float* add, float* out, int T, int K, int F, int H,
-                     int top, int E, int gated, hipStream_t s) {
+                     int top, int E, int kind, int weigh_input, hipStream_t s) {
   if (T == 0) return 0;
   KVCM_REQUIRE(T > 0 && top > 0 && H > 0 && ldh >= K, "moe_grouped: bad sizes");
   KVCM_REQUIRE(kvcm_moe_grouped_supported(K, F, E), "moe_grouped: sizes K=%d F=%d experts=%d are not supported", K, F, E);
@@ -252,21 +251,25 @@ int kvcm_moe_grouped(const void* h, int ldh, const void* w_up, const void* w_dow
                    reinterpret_cast<uintptr_t>(w_down) % 16 == 0 && reinterpret_cast<uintptr_t>(act) % 16 == 0,
                "moe_grouped: operands must be 16-byte aligned");
   const int n = T * top, max_tiles = kvcm_moe_grouped_max_tiles(n, E);
-  KVCM_REQUIRE(!gated || F % 16 == 0, "moe_grouped: gated experts of %d columns are not supported (a multiple of 16)", F);
-  const int up_rows = gated ? 2 * F : F;
+  KVCM_REQUIRE(kind >= 0 && kind <= 2, "moe_grouped: unknown kind of experts %d (0 relu2, 1 silu gated, 2 gelu)", kind);
+  KVCM_REQUIRE(kind != 1 || F % 16 == 0, "moe_grouped: gated experts of %d columns are not supported (a multiple of 16)", F);
+  const int up_rows = kind == 1 ? 2 * F : F;
+  const float *up_weight = weigh_input ? weight : nullptr, *down_weight = weigh_input ? nullptr : weight;
   const int up_blocks = (up_rows + kGN - 1) / kGN, down_blocks = (H + kGN - 1) / kGN;
   const long long up_grid = static_cast<long long>(max_tiles) * ((up_blocks + 7) / 8) * 8;
   const long long down_grid = static_cast<long long>(max_tiles) * ((down_blocks + 7) / 8) * 8;
   KVCM_REQUIRE(up_grid < (1ll << 31) && down_grid < (1ll << 31), "moe_grouped: too many tiles");
   moe_group_kernel<<<1, 1024, 2 * E * sizeof(int), s>>>(chosen, n, E, order, tiles, max_tiles);
-  if (gated)
-    moe_grouped_kernel<kUpGated><<<static_cast<unsigned>(up_grid), 256, 0, s>>>(
-        static_cast<const uint16_t*>(h), ldh, static_cast<const uint16_t*>(w_up), order, tiles, top, act, nullptr, up_rows, K, up_blocks);
-  else
-    moe_grouped_kernel<kUp><<<static_cast<unsigned>(up_grid), 256, 0, s>>>(
-        static_cast<const uint16_t*>(h), ldh, static_cast<const uint16_t*>(w_up), order, tiles, top, act, nullptr, F, K, up_blocks);
+#define KVCM_GROUPED_UP(MODE)                                                                                              \
+  moe_grouped_kernel<MODE><<<static_cast<unsigned>(up_grid), 256, 0, s>>>(static_cast<const uint16_t*>(h), ldh,            \
+                                                                          static_cast<const uint16_t*>(w_up), order, tiles, \
+                                                                          top, act, up_weight, up_rows, K, up_blocks)
+  if (kind == 1) KVCM_GROUPED_UP(kUpGated);
+  else if (kind == 2) KVCM_GROUPED_UP(kUpGelu);
+  else KVCM_GROUPED_UP(kUp);
+#undef KVCM_GROUPED_UP
   moe_grouped_kernel<kDown><<<static_cast<unsigned>(down_grid), 256, 0, s>>>(
-      static_cast<const uint16_t*>(act), F, static_cast<const uint16_t*>(w_down), order, tiles, top, y, weight, H, F, down_blocks);
+      static_cast<const uint16_t*>(act), F, static_cast<const uint16_t*>(w_down), order, tiles, top, y, down_weight, H, F, down_blocks);
   const long long total = static_cast<long long>(T) * H;
   const long long blocks = (total + 255) / 256;
   moe_combine_kernel<<<static_cast<unsigned>(blocks > 16384 ? 16384 : blocks), 256, 0, s>>>(y, add, out, total, H, top);

@@ -6,7 +6,7 @@
 //                  the un-added slices of a product that was split along K: they are added here, in their order.  With a
 //                  row gather (the model's last norm, on the rows whose logits are wanted) nothing is written back.
 //   group_norm_gate  a gate before a norm: v = y * silu(z), then groups of consecutive columns of v are divided by their
-//                  root mean square and weighted.
+//                  root mean square and weighted; or (after) the norm first, v = y, and then the factor sigmoid(z).
 //
 // All arithmetic is 32-bit; a row's result is one fixed sequence of operations on that row alone.
 #include "common.h"
@@ -137,7 +137,7 @@ __global__ void __launch_bounds__(kTermThreads)
 template <class TO>
 __global__ void __launch_bounds__(kTermThreads)
     group_norm_gate_kernel(const float* __restrict__ y, int ldy, const float* __restrict__ z, int ldz, const float* __restrict__ w,
-                           TO* __restrict__ out, int ldo, int size, float eps) {
+                           TO* __restrict__ out, int ldo, int size, float eps, int after) {
   __shared__ float scratch[kTermThreads / kWave];
   constexpr int kHeld = 16;
   const int row = blockIdx.x, c0 = blockIdx.y * size;
@@ -145,22 +145,24 @@ __global__ void __launch_bounds__(kTermThreads)
   const float* zr = z + size_t(row) * ldz + c0;
   TO* o = out + size_t(row) * ldo + c0;
   auto value = [&](int i) {
+    if (after) return yr[i];
     const float g = zr[i];
     return yr[i] * (g / (1.0f + expf(-g)));
   };
   if (size <= kHeld * kTermThreads) {
-    float v[kHeld], ss = 0.f;
+    float v[kHeld], gate[kHeld], ss = 0.f;
 #pragma unroll
     for (int j = 0; j < kHeld; ++j) {
       const int i = threadIdx.x + j * kTermThreads;
       v[j] = i < size ? value(i) : 0.f;
+      gate[j] = (after && i < size) ? 1.0f / (1.0f + expf(-zr[i])) : 1.f;
       ss = fmaf(v[j], v[j], ss);
     }
     const float inv = 1.0f / sqrtf(terms_block_sum(ss, scratch) / float(size) + eps);
 #pragma unroll
     for (int j = 0; j < kHeld; ++j) {
       const int i = threadIdx.x + j * kTermThreads;
-      if (i < size) store_f(o + i, v[j] * inv * w[c0 + i]);
+      if (i < size) store_f(o + i, v[j] * inv * w[c0 + i] * gate[j]);
     }
     return;
   }
@@ -170,7 +172,8 @@ __global__ void __launch_bounds__(kTermThreads)
     ss = fmaf(v, v, ss);
   }
   const float inv = 1.0f / sqrtf(terms_block_sum(ss, scratch) / float(size) + eps);
-  for (int i = threadIdx.x; i < size; i += kTermThreads) store_f(o + i, value(i) * inv * w[c0 + i]);
+  for (int i = threadIdx.x; i < size; i += kTermThreads)
+    store_f(o + i, value(i) * inv * w[c0 + i] * (after ? 1.0f / (1.0f + expf(-zr[i])) : 1.f));
 }
 
 }  // namespace kvcm
@@ -213,15 +216,15 @@ int kvcm_stream_terms(float* x, const float* a, int a_splits, float a_factor, co
 
 // y, z [T, >= groups * size] 32-bit rows; w [groups * size]; out [T, >= groups * size] in out_dtype
 int kvcm_group_norm_gate(const float* y, int ldy, const float* z, int ldz, const float* w, void* out, int out_dtype, int ldo, int T,
-                         int groups, int size, float eps, hipStream_t s) {
+                         int groups, int size, float eps, int after, hipStream_t s) {
   if (T == 0) return 0;
   KVCM_REQUIRE(T > 0 && groups > 0 && size > 0 && y && z && w && out, "group_norm_gate: bad sizes T=%d groups=%d size=%d", T, groups, size);
   KVCM_REQUIRE(groups <= 65535 && ldy >= groups * size && ldz >= groups * size && ldo >= groups * size, "group_norm_gate: row strides too small");
   const dim3 grid(T, groups);
   if (out_dtype == kF32)
-    group_norm_gate_kernel<float><<<grid, kTermThreads, 0, s>>>(y, ldy, z, ldz, w, static_cast<float*>(out), ldo, size, eps);
+    group_norm_gate_kernel<float><<<grid, kTermThreads, 0, s>>>(y, ldy, z, ldz, w, static_cast<float*>(out), ldo, size, eps, after);
   else if (out_dtype == kBF16)
-    group_norm_gate_kernel<bf16_t><<<grid, kTermThreads, 0, s>>>(y, ldy, z, ldz, w, static_cast<bf16_t*>(out), ldo, size, eps);
+    group_norm_gate_kernel<bf16_t><<<grid, kTermThreads, 0, s>>>(y, ldy, z, ldz, w, static_cast<bf16_t*>(out), ldo, size, eps, after);
   else KVCM_REQUIRE(false, "group_norm_gate: unknown output dtype %d", out_dtype);
   return launch_status("group_norm_gate");
 }

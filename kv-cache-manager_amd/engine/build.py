@@ -41,14 +41,20 @@ def read_model_config(model_dir):
     return arch, arch.config_class.from_dict(raw)
 
 
-def within_max_position(ec: EngineConfig, max_position: int) -> EngineConfig:
+def within_max_position(ec: EngineConfig, max_position: int, fixed: bool = False) -> EngineConfig:
     """The model's own length limit against the engine's.  The reference carries max_pos in its
     weights header and never looks at it (src/model/weights.cpp:24-40): positions are rotated on the
     fly, so any length computes.  Here the engine's max_seq_len is cut down to the model's
     max_position (0: the architecture states none), with one line on stderr, unless the option
-    ``beyond_max_position`` says that running past it is meant (replay of given traces does)."""
-    if max_position <= 0 or ec.max_seq_len <= max_position or ec.beyond_max_position:
+    ``beyond_max_position`` says that running past it is meant (replay of given traces does).  ``fixed``: the model has a
+    learned vector for each of its positions and none beyond them; the option does not lift that."""
+    if max_position <= 0 or ec.max_seq_len <= max_position or (ec.beyond_max_position and not fixed):
         return ec
+    if fixed:
+        if not ec.beyond_max_position:
+            print(f"[kvcm] max_seq_len {ec.max_seq_len} exceeds the model's {max_position} learned positions: sequences end there",
+                  file=sys.stderr, flush=True)
+        return dataclasses.replace(ec, max_seq_len=max_position)
     print(f"[kvcm] max_seq_len {ec.max_seq_len} exceeds the model's max_position_embeddings {max_position}: "
           f"sequences end at {max_position} tokens (EngineConfig.beyond_max_position=True lifts this)", file=sys.stderr, flush=True)
     return dataclasses.replace(ec, max_seq_len=max_position)
@@ -72,7 +78,7 @@ def build_runner(model_dir: Optional[str] = None, engine_config: Optional[Engine
             raise ValueError("give a model folder, or architecture + model_config + tensors")
         arch, cfg, source = ARCHITECTURES.get(architecture), model_config, DictSource(tensors)
     spec = arch.build_spec(cfg)
-    ec = within_max_position(ec, spec.max_position)
+    ec = within_max_position(ec, spec.max_position, spec.max_position_fixed)
     model = Model(spec, BuildContext(dtype, dev, spec.hidden_size, ec.block_size, ops))
     try:
         weight_bytes = load_weights(model, source, dtype, dev)

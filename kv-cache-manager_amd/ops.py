@@ -45,7 +45,7 @@ def _declare(lib):
     fn("kvcm_attention_generic_info", i, vp)
     fn("kvcm_attention_decode_fused_info", i, i, i, vp)
     fn("kvcm_gemm_skinny_swiglu_supported", i, i, i)
-    fn("kvcm_gemm_skinny_swiglu", vp, vp, vp, i, i, i, i, i, i, i, vp)
+    fn("kvcm_gemm_skinny_swiglu", vp, vp, vp, i, i, i, i, i, i, i, f, vp)
     fn("kvcm_gemm_skinny_splits", i, i, i)
     fn("kvcm_gemm_skinny_waves", i, i, i, i, i)
     fn("kvcm_gemm_skinny_swiglu_normed_preferred", i, i, i)
@@ -89,8 +89,8 @@ def _declare(lib):
     fn("kvcm_gemm8_supported", i, i, i)
     fn("kvcm_gemm8", vp, i, vp, i, i, i, i, vp, i, f, vp, i, i, i, vp)
     fn("kvcm_gemm8_residual_norm", vp, i, vp, i, i, i, i, vp, vp, i, vp, vp, vp)
-    fn("kvcm_embed_scaled", vp, vp, i, vp, i, i, i, f, vp)
-    fn("kvcm_gated_act", vp, i, vp, vp, i, vp, i, i, i, i, i, vp)
+    fn("kvcm_embed_scaled", vp, vp, i, vp, i, i, i, f, vp, vp, i, vp)
+    fn("kvcm_gated_act", vp, i, vp, vp, i, vp, i, i, i, i, i, f, vp)
     fn("kvcm_rmsnorm_chain", vp, vp, i, vp, i, C.c_longlong, vp, vp, f, vp, vp, vp, vp, i, i, i, f, vp)
     fn("kvcm_head_norm_gate", vp, i, vp, i, vp, vp, i, i, i, i, i, f, i, vp)
     fn("kvcm_short_conv", vp, i, vp, vp, vp, vp, vp, i, i, vp, vp, vp, vp, vp, vp, i, i, i, i, i, vp)
@@ -112,19 +112,19 @@ def _declare(lib):
     fn("kvcm_mlstm_scan", vp, i, vp, i, vp, i, vp, i, vp, i, vp, vp, f, f, vp, vp, vp, i, vp, vp, vp, vp, vp, vp, i, i, i, i, i, i, vp)
     fn("kvcm_moe_route", vp, i, i, C.c_longlong, i, i, i, f, vp, vp, i, vp)
     fn("kvcm_moe_table_route", vp, vp, i, i, i, vp, vp, i, vp)
-    fn("kvcm_moe_up", vp, i, i, vp, vp, vp, i, i, i, i, i, i, vp)
+    fn("kvcm_moe_up", vp, i, i, vp, vp, vp, i, i, i, i, i, i, vp, vp)
     fn("kvcm_moe_down", vp, i, vp, vp, vp, vp, vp, i, i, i, i, i, vp)
     fn("kvcm_moe_grouped_supported", i, i, i)
     fn("kvcm_moe_grouped_max_tiles", i, i)
-    fn("kvcm_moe_grouped", vp, i, vp, vp, vp, vp, vp, vp, vp, vp, vp, vp, i, i, i, i, i, i, i, vp)
+    fn("kvcm_moe_grouped", vp, i, vp, vp, vp, vp, vp, vp, vp, vp, vp, vp, i, i, i, i, i, i, i, i, vp)
     fn("kvcm_pool_update", vp, vp, i, vp, vp, vp, i, vp, vp, vp, i, i, i, i, i, i, i, vp)
-    fn("kvcm_attention_window_pool", vp, i, i, vp, i, vp, vp, vp, vp, vp, i, vp, vp, vp, vp, vp, i, i, i, i, i, i, i, f, i, i, i, i, f, i, i, f, vp)
+    fn("kvcm_attention_window_pool", vp, i, i, vp, i, vp, vp, vp, vp, vp, i, vp, vp, vp, vp, vp, i, i, i, i, i, i, i, f, i, i, i, i, f, i, i, vp, i, f, vp)
     fn("kvcm_attention_window_pool_tiles_supported", i, i, i)
-    fn("kvcm_attention_window_pool_tiles", vp, i, vp, i, vp, vp, vp, vp, vp, i, vp, vp, vp, vp, vp, i, i, i, i, i, i, i, i, f, i, i, i, i, f, i, i, f, vp)
+    fn("kvcm_attention_window_pool_tiles", vp, i, vp, i, vp, vp, vp, vp, vp, i, vp, vp, vp, vp, vp, i, i, i, i, i, i, i, i, f, i, i, i, i, f, i, i, vp, i, f, vp)
     fn("kvcm_selective_scan", vp, i, i, vp, i, vp, vp, i, i, i, vp, vp, vp, i, vp, i, vp, vp, vp, vp, i, i, i, i, i, i, vp, C.c_longlong, i, vp)
     fn("kvcm_stream_terms", vp, vp, i, f, vp, i, f, vp, i, f, C.c_longlong, vp, vp, vp, vp, vp, i, i, i, f, vp)
-    fn("kvcm_group_norm_gate", vp, i, vp, i, vp, vp, i, i, i, i, i, f, vp)
-    fn("kvcm_gated_state", vp, i, vp, i, vp, i, vp, i, vp, i, vp, vp, vp, i, vp, i, vp, vp, vp, vp, i, i, i, i, i, i, i, i, vp, C.c_longlong, vp)
+    fn("kvcm_group_norm_gate", vp, i, vp, i, vp, vp, i, i, i, i, i, f, i, vp)
+    fn("kvcm_gated_state", vp, i, vp, i, vp, i, vp, i, vp, i, vp, vp, vp, vp, i, i, vp, i, vp, vp, vp, vp, i, i, i, i, i, i, i, i, vp, C.c_longlong, vp)
     lib.kvcm_gated_state_carry_floats.restype = C.c_longlong
     lib.kvcm_gated_state_carry_floats.argtypes = [i] * 7
     fn("kvcm_scan_prepare", vp, i, vp, vp, i, i, i, vp)
@@ -647,11 +647,13 @@ def gemm(x, w, out, scratch=None, keep_partial=False, tuning=None):
     return out
 
 
-def gemm_swiglu(x, w_gate_up, out):
-    """out[M, I] = swiglu(x[M, K] @ w_gate_up[2 I, K]^T) in one launch, or False when this shape
+def gemm_swiglu(x, w_gate_up, out, limit=0.0):
+    """out[M, I] = swiglu(x[M, K] @ w_gate_up[2 I, K]^T), or with ``limit`` > 0 its form with limits (``gated_act``'s "clamped"), in one launch, or False when this shape
     has no fused kernel (then the caller runs the product and ``swiglu`` one after the other:
     the same values up to the order of the sums)."""
     if isinstance(x, NormedRows):
+        if limit > 0:
+            return False          # (the kernels that take rows whose norm is still to be applied know silu only)
         M, K = x.shape
         I = out.shape[1]
         _dev(x.xg, x.ss, w_gate_up, out)
@@ -679,7 +681,7 @@ def gemm_swiglu(x, w_gate_up, out):
             and lib().kvcm_gemm_skinny_swiglu_supported(M, I, K)):
         return False
     _call("kvcm_gemm_skinny_swiglu", _ptr(x), _ptr(w_gate_up), _ptr(out), _DT[out.dtype], M, I, K, x.stride(0),
-                                         w_gate_up.stride(0), out.stride(0), _stream())
+                                         w_gate_up.stride(0), out.stride(0), float(limit), _stream())
     return True
 
 
@@ -966,7 +968,9 @@ def sample(logits, out, temperature=None, seeds=None, request_ids=None, token_in
 
 
 # ------------------------------------------------------------- parts of other sequence models
-GATE_ACTIVATIONS = {"silu": 0, "relu": 1, "gelu_tanh": 2}
+ACTIVATIONS = {"silu": 0, "relu": 1, "gelu_tanh": 2, "gelu": 3}      # gelu: the exact form, by the error function
+GATE_ACTIVATIONS = {**ACTIVATIONS, "clamped": 4}
+EXPERT_KINDS = {"relu2": 0, "silu_gated": 1, "gelu": 2}
 
 
 def _f32(t, name, n=None):
@@ -982,18 +986,25 @@ def _f32rows(t, name, cols):
           f"{name} must be float32 rows of at least {cols} columns")
 
 
-def embed_scaled(ids, table, out, factor):
-    """out[t, :] = float(table[ids[t], :]) * factor."""
+def embed_scaled(ids, table, out, factor, positions=None, pos_table=None):
+    """out[t, :] = float(table[ids[t], :]) * factor (+ float(pos_table[positions[t], :]), a vector per position as it is)."""
     _dev(ids, table, out)
     T, H = out.shape
     _i32(ids, "ids", T)
     _need(table.dim() == 2 and table.shape[1] == H and table.is_contiguous(), "embedding table must be [V, H]")
     _need(out.dtype == torch.float32 and out.is_contiguous(), "residual stream must be contiguous float32")
-    _call("kvcm_embed_scaled", _ptr(ids), _ptr(table), _DT[table.dtype], _ptr(out), T, H, table.shape[0], float(factor), _stream())
+    if pos_table is not None:
+        _need(positions is not None, "embed_scaled: vectors by position need the positions")
+        _i32(positions, "positions", T)
+        _need(pos_table.dim() == 2 and pos_table.shape[1] == H and pos_table.is_contiguous() and pos_table.is_cuda
+              and pos_table.dtype == table.dtype, "the table of positions must be [P, H] of the embedding table's dtype")
+    _call("kvcm_embed_scaled", _ptr(ids), _ptr(table), _DT[table.dtype], _ptr(out), T, H, table.shape[0], float(factor),
+          _ptr(positions) if pos_table is not None else 0, _ptr(pos_table), pos_table.shape[0] if pos_table is not None else 0, _stream())
 
 
-def gated_act(gate_up, out, activation, bias=None, row_gate=None):
-    """out[T, I] = act(gate) * up for 32-bit rows [gate (I) | up (I)]; act: "silu", "relu" or "gelu_tanh".  ``bias`` (float32
+def gated_act(gate_up, out, activation, bias=None, row_gate=None, limit=0.0):
+    """out[T, I] = act(gate) * up for 32-bit rows [gate (I) | up (I)]; act: "silu", "relu", "gelu_tanh" or "gelu"; or "clamped":
+    g = min(gate, limit), u = up held within [-limit, limit], out = g * sigmoid(1.702 g) * (u + 1).  ``bias`` (float32
     [2I]): added to the rows first.  ``row_gate`` (float32 rows, column 0 is read): the result times sigmoid(row_gate[t, 0])."""
     T, I = out.shape
     _f32rows(gate_up, "gate_up", 2 * I)
@@ -1005,7 +1016,7 @@ def gated_act(gate_up, out, activation, bias=None, row_gate=None):
         _f32rows(row_gate, "row_gate", 1)
         _need(row_gate.shape[0] >= T, "gated_act: fewer gates than rows")
     _call("kvcm_gated_act", _ptr(gate_up), gate_up.stride(0), _ptr(bias), _ptr(row_gate), row_gate.stride(0) if row_gate is not None else 0, _ptr(out), _DT[out.dtype], out.stride(0), T, I,
-          GATE_ACTIVATIONS[activation], _stream())
+          GATE_ACTIVATIONS[activation], float(limit or 0.0), _stream())
 
 
 class NormedBranches:
@@ -1217,16 +1228,25 @@ def pool_update(kcache, vcache, pk, pv, tables, table_stride, row_seq, positions
           _ptr(row_seq), _ptr(positions), _ptr(slots), rows, nkv, d, dv, B, P, E, _stream())
 
 
+def _sink(sink, nh):
+    """An attention's ``sink`` argument -> (is there one, its scores per head or None)."""
+    if not torch.is_tensor(sink):
+        return (1 if sink else 0), None
+    _f32(sink, "sink", nh)
+    return 1, sink
+
+
 def attention_window_pool(q, out, kcache, vcache, pk, pv, tables, table_stride, row_seq, ctx_lens, nh, nkv, d, dv, scale,
                           window, P, head_scale=None, rows=None, keep_first=0, softcap=0.0, dist_slope=None, gate=None, chunk=0, sink=False,
-                          out_scale=1.0):
+                          out_scale=1.0, gate_heads=False):
     """out[r, h] = softmax over the last ``window`` tokens, the sequence's first ``keep_first`` tokens and the pooled
     blocks of P tokens before the window (window 0: every token, no blocks) of (q . k) * scale * head_scale[h], times the
     values.  ``softcap`` c > 0: the scores are capped first, c tanh(score / c).  ``dist_slope`` (float32 [nh]): a bias that
     grows with the distance is taken off the scores, slope[h] * (query position - key position).  ``gate`` (float32 rows of
     >= nh*dv): the output is multiplied element by element with sigmoid(gate) before it is stored.  ``chunk`` > 0 (window 0):
-    a row at position i sees the tokens j <= i with j // chunk == i // chunk.  ``sink``: one is added to the softmax's
-    denominator (a key of score 0 without a value).  ``out_scale``: a factor on the output."""
+    a row at position i sees the tokens j <= i with j // chunk == i // chunk.  ``sink``: True: one is added to the softmax's
+    denominator (a key of score 0 without a value); float32 [nh]: exp(sink[h]) is.  ``gate_heads``: the gate is one logit per
+    head, rows of >= nh.  ``out_scale``: a factor on the output."""
     _dev(q, out, kcache, vcache, tables, row_seq, ctx_lens)
     _rows2d(q, "q")
     _rows2d(out, "out")
@@ -1237,15 +1257,16 @@ def attention_window_pool(q, out, kcache, vcache, pk, pv, tables, table_stride, 
     _f32(head_scale, "head_scale", nh)
     _f32(dist_slope, "dist_slope", nh)
     if gate is not None:
-        _f32rows(gate, "gate", nh * dv)
+        _f32rows(gate, "gate", nh if gate_heads else nh * dv)
         _need(gate.shape[0] >= T, "attention_window_pool: the gate has fewer rows than the step")
+    sink, sink_logit = _sink(sink, nh)
     _i32(row_seq, "row_seq", T)
     _i32(ctx_lens, "ctx_lens", T)
     _i32(tables, "tables")
     _call("kvcm_attention_window_pool", _ptr(q), _DT[q.dtype], q.stride(0), _ptr(out), out.stride(0), _ptr(kcache), _ptr(vcache),
           _ptr(pk), _ptr(pv), _ptr(tables), table_stride, _ptr(row_seq), _ptr(ctx_lens), _ptr(head_scale), _ptr(dist_slope), _ptr(gate),
           gate.stride(0) if gate is not None else 0, T, nh, nkv, d, dv,
-          B, float(scale), int(window), int(P), E, int(keep_first), float(softcap or 0.0), int(chunk), 1 if sink else 0, float(out_scale), _stream())
+          B, float(scale), int(window), int(P), E, int(keep_first), float(softcap or 0.0), int(chunk), sink, _ptr(sink_logit), 1 if gate_heads else 0, float(out_scale), _stream())
 
 
 def attention_window_pool_tiles_supported(d, dv, dtype, block_size):
@@ -1255,7 +1276,7 @@ def attention_window_pool_tiles_supported(d, dv, dtype, block_size):
 
 def attention_window_pool_tiles(q, out, kcache, vcache, pk, pv, tables, table_stride, run_start, seq_start, num_seqs, max_run,
                                 nh, nkv, d, dv, scale, window, P, head_scale=None, keep_first=0, softcap=0.0, dist_slope=None, gate=None,
-                                chunk=0, sink=False, out_scale=1.0):
+                                chunk=0, sink=False, out_scale=1.0, gate_heads=False):
     """``attention_window_pool`` for steps whose sequences run several consecutive positions: 64 rows of a run and one
     head per workgroup on the matrix cores (bfloat16 only).  Every row of every run is computed, single rows too."""
     _dev(q, out, kcache, vcache, tables, run_start, seq_start)
@@ -1267,15 +1288,17 @@ def attention_window_pool_tiles(q, out, kcache, vcache, pk, pv, tables, table_st
     _f32(head_scale, "head_scale", nh)
     _f32(dist_slope, "dist_slope", nh)
     if gate is not None:
-        _f32rows(gate, "gate", nh * dv)
+        _f32rows(gate, "gate", nh if gate_heads else nh * dv)
         _need(gate.shape[0] >= out.shape[0], "attention_window_pool_tiles: the gate has fewer rows than the output")
+    sink, sink_logit = _sink(sink, nh)
     _i32(run_start, "run_start", num_seqs + 1)
     _i32(seq_start, "seq_start", num_seqs)
     _i32(tables, "tables")
     _call("kvcm_attention_window_pool_tiles", _ptr(q), q.stride(0), _ptr(out), out.stride(0), _ptr(kcache), _ptr(vcache), _ptr(pk),
           _ptr(pv), _ptr(tables), table_stride, _ptr(run_start), _ptr(seq_start), _ptr(head_scale), _ptr(dist_slope), _ptr(gate),
           gate.stride(0) if gate is not None else 0, num_seqs, max_run, nh, nkv,
-          d, dv, B, float(scale), int(window), int(P), E, int(keep_first), float(softcap or 0.0), int(chunk), 1 if sink else 0, float(out_scale), _stream())
+          d, dv, B, float(scale), int(window), int(P), E, int(keep_first), float(softcap or 0.0), int(chunk), sink, _ptr(sink_logit), 1 if gate_heads else 0,
+          float(out_scale), _stream())
 
 
 SCAN_PIECE = 128      # rows of a piece when long runs are walked in pieces
@@ -1572,7 +1595,7 @@ def gemm_heads(x, w, out, gate=None, rows=None):
 
 def act_rows(x, out, activation):
     """out[T, I] = act(x[T, :I]) for 32-bit rows (a tensor, or PartialSums whose slices are added first); act: "silu",
-    "relu" or "gelu_tanh"."""
+    "relu", "gelu_tanh" or "gelu"."""
     T, I = out.shape
     _rows2d(out, "out")
     splits, stride = 1, 0
@@ -1586,8 +1609,8 @@ def act_rows(x, out, activation):
         _need(x.shape[0] >= T, "act_rows: the rows do not agree")
         ld = x.stride(0)
     _need(out.is_cuda, "act_rows: the output must live on the GPU")
-    _need(activation in GATE_ACTIVATIONS, f"unknown activation {activation!r} ({sorted(GATE_ACTIVATIONS)})")
-    _call("kvcm_act_rows", _ptr(x), ld, splits, stride, _ptr(out), _DT[out.dtype], out.stride(0), T, I, GATE_ACTIVATIONS[activation], _stream())
+    _need(activation in ACTIVATIONS, f"unknown activation {activation!r} ({sorted(ACTIVATIONS)})")
+    _call("kvcm_act_rows", _ptr(x), ld, splits, stride, _ptr(out), _DT[out.dtype], out.stride(0), T, I, ACTIVATIONS[activation], _stream())
     return out
 
 
@@ -1613,11 +1636,13 @@ def mlstm_scan(q, k, v, gate_in, gate_keep, in_bias, keep_bias, cap, q_scale, co
     return o
 
 
-def moe_route(logits, experts, top, chosen, weight, rows=None, over_chosen=False, factor=1.0):
+def moe_route(logits, experts, top, chosen, weight, rows=None, over_chosen=False, factor=1.0, sigmoid=False):
     """chosen[T, top] (int32) and weight[T, top] (float32): the ``top`` experts with the largest softmax scores over all
     ``experts`` of each row's 32-bit router logits, best first, with those scores; ``over_chosen``: with the softmax over
     the chosen logits alone instead (the weights of a row add up to one).  ``logits`` may be PartialSums (a router product
-    that was split along K): the slices are added as they are read.  ``factor``: a constant on the weights."""
+    that was split along K): the slices are added as they are read.  ``factor``: a constant on the weights.  ``sigmoid``: a
+    score is sigmoid of its own logit (which chooses the same experts), and the weights are those scores."""
+    _need(not (over_chosen and sigmoid), "moe_route: one kind of weights")
     T = chosen.shape[0] if rows is None else rows
     splits, stride = 1, 0
     if isinstance(logits, PartialSums):
@@ -1632,7 +1657,7 @@ def moe_route(logits, experts, top, chosen, weight, rows=None, over_chosen=False
           "chosen must be int32 [T, top]")
     _need(weight.dtype == torch.float32 and weight.is_contiguous() and weight.is_cuda and tuple(weight.shape) == tuple(chosen.shape),
           "weight must be float32 [T, top]")
-    _call("kvcm_moe_route", _ptr(logits), ld, splits, stride, experts, top, 1 if over_chosen else 0, float(factor), _ptr(chosen), _ptr(weight),
+    _call("kvcm_moe_route", _ptr(logits), ld, splits, stride, experts, top, 1 if over_chosen else 2 if sigmoid else 0, float(factor), _ptr(chosen), _ptr(weight),
           T, _stream())
 
 
@@ -1656,11 +1681,17 @@ def _expert_shapes(w_up, w_down, gated):
     return E, F, K
 
 
-def moe_rows(h, w_up, w_down, chosen, weight, act, out, gated=False, add=None):
+def _expert_kind(gated, activation):
+    _need(activation in ("relu2", "gelu"), f"experts without a gate: unknown activation {activation!r} (relu2 | gelu)")
+    return EXPERT_KINDS["silu_gated" if gated else activation]
+
+
+def moe_rows(h, w_up, w_down, chosen, weight, act, out, gated=False, add=None, activation="relu2", weigh_input=False):
     """out[T, H] (float32) = sum over a row's chosen experts e of weight * W_down[e] square(relu(W_up[e] h)), a row at a
     time, reading only the chosen experts.  h [T, K]; w_up [E, F, K]; w_down [E, H, F]; act: work memory [T * top, F].
     ``gated``: w_up is ``interleave_gate_up`` of the experts' gate and up matrices and the activation is
-    silu(W_gate h) * (W_up h).  ``add`` (float32 [T, H]): out = add + the sum."""
+    silu(W_gate h) * (W_up h); otherwise ``activation`` may be "gelu" instead of "relu2".  ``weigh_input``: the weights are
+    factors on what the experts read, not on what they give.  ``add`` (float32 [T, H]): out = add + the sum."""
     T, K = h.shape
     E, F, _ = _expert_shapes(w_up, w_down, gated)
     H, top = w_down.shape[1], chosen.shape[1]
@@ -1674,8 +1705,9 @@ def moe_rows(h, w_up, w_down, chosen, weight, act, out, gated=False, add=None):
     _need(out.dtype == torch.float32 and out.is_contiguous() and tuple(out.shape) == (T, H), "out must be float32 [T, H]")
     _need(chosen.dtype == torch.int32 and chosen.is_contiguous() and chosen.shape[0] >= T, "chosen must be int32 [T, top]")
     _need(weight.dtype == torch.float32 and weight.is_contiguous() and tuple(weight.shape) == tuple(chosen.shape), "weight must match chosen")
-    _call("kvcm_moe_up", _ptr(h), _DT[h.dtype], h.stride(0), _ptr(w_up), _ptr(chosen), _ptr(act), T, K, F, top, E, 1 if gated else 0, _stream())
-    _call("kvcm_moe_down", _ptr(act), _DT[act.dtype], _ptr(w_down), _ptr(chosen), _ptr(weight), _ptr(add), _ptr(out), T, F, H, top, E, _stream())
+    _call("kvcm_moe_up", _ptr(h), _DT[h.dtype], h.stride(0), _ptr(w_up), _ptr(chosen), _ptr(act), T, K, F, top, E,
+          _expert_kind(gated, activation), _ptr(weight) if weigh_input else 0, _stream())
+    _call("kvcm_moe_down", _ptr(act), _DT[act.dtype], _ptr(w_down), _ptr(chosen), 0 if weigh_input else _ptr(weight), _ptr(add), _ptr(out), T, F, H, top, E, _stream())
     return out
 
 
@@ -1689,7 +1721,7 @@ def moe_grouped_tiles(pairs, E):
     return 3 * lib().kvcm_moe_grouped_max_tiles(int(pairs), int(E)) + 1
 
 
-def moe_grouped(h, w_up, w_down, chosen, weight, order, tiles, act, y, out, gated=False, add=None):
+def moe_grouped(h, w_up, w_down, chosen, weight, order, tiles, act, y, out, gated=False, add=None, activation="relu2", weigh_input=False):
     """As ``moe_rows``, for steps with many rows (bfloat16): the (row, slot) pairs grouped by expert and multiplied in tiles
     on the matrix cores.  Work memory: order int32 [T * top], tiles int32 [moe_grouped_tiles], act [T * top, F],
     y float32 [T * top, H]."""
@@ -1710,7 +1742,7 @@ def moe_grouped(h, w_up, w_down, chosen, weight, order, tiles, act, y, out, gate
     _i32(order, "order", T * top)
     _i32(tiles, "tiles", moe_grouped_tiles(T * top, E))
     _call("kvcm_moe_grouped", _ptr(h), h.stride(0), _ptr(w_up), _ptr(w_down), _ptr(chosen), _ptr(weight), _ptr(order), _ptr(tiles),
-          _ptr(act), _ptr(y), _ptr(add), _ptr(out), T, K, F, H, top, E, 1 if gated else 0, _stream())
+          _ptr(act), _ptr(y), _ptr(add), _ptr(out), T, K, F, H, top, E, _expert_kind(gated, activation), 1 if weigh_input else 0, _stream())
     return out
 
 
@@ -1735,6 +1767,11 @@ class StreamTerms:
         if isinstance(value, BiasedOutput):
             return cls([(value.value, 1.0)], value.bias)
         return cls([(value, 1.0)])
+
+    def only(self):
+        """The one term's value, where that is all there is (a sublayer's plain output)."""
+        _need(len(self.terms) == 1 and self.terms[0][1] == 1.0 and self.bias is None, "StreamTerms: more than one plain term")
+        return self.terms[0][0]
 
     def plus(self, other):
         other = StreamTerms.of(other)
@@ -1780,9 +1817,9 @@ def stream_terms(x, eps, add=None, again=None, weight=None, out=None, rows=None)
     return out
 
 
-def group_norm_gate(y, z, weight, out, groups, size, eps):
-    """out[t, g*size + i] = n(y * silu(z))[i of group g] * weight, n: division by the group's own root mean square; y, z
-    float32 rows of groups*size, out rows of any stored dtype."""
+def group_norm_gate(y, z, weight, out, groups, size, eps, after=False):
+    """out[t, g*size + i] = n(y * silu(z))[i of group g] * weight, n: division by the group's own root mean square; ``after``:
+    n(y)[i of group g] * weight * sigmoid(z).  y, z float32 rows of groups*size, out rows of any stored dtype."""
     T = out.shape[0]
     _f32rows(y, "y", groups * size)
     _f32rows(z, "z", groups * size)
@@ -1790,7 +1827,7 @@ def group_norm_gate(y, z, weight, out, groups, size, eps):
     _rows2d(out, "out")
     _need(y.shape[0] >= T and z.shape[0] >= T and out.shape[1] >= groups * size and out.is_cuda, "group_norm_gate: shapes do not agree")
     _call("kvcm_group_norm_gate", _ptr(y), y.stride(0), _ptr(z), z.stride(0), _ptr(weight), _ptr(out), _DT[out.dtype], out.stride(0), T,
-          groups, size, float(eps), _stream())
+          groups, size, float(eps), 1 if after else 0, _stream())
     return out
 
 
@@ -1806,27 +1843,35 @@ def gated_state_carry_floats(rows, seqs, heads, dk, dv, delta, piece=None):
     return int(lib().kvcm_gated_state_carry_floats(rows, seqs, heads, dk, dv, 1 if delta else 0, piece or gated_state_piece(dk)))
 
 
-def gated_state(q, k, v, a, dt_bias, a_log, o, state, step, heads, groups, dk, dv, b=None, d_skip=None, carry=None, piece=None):
+def gated_state(q, k, v, a, dt_bias, a_log, o, state, step, heads, groups, dk, dv, b=None, d_skip=None, carry=None, piece=None,
+                decay=None, silu_in=False):
     """A matrix state per head with one decay per head and token over the step's runs (csrc/hip/gated_state.hip).  q, k
     [T, groups*dk], v [T, heads*dv], a [T, heads]: float32 rows; state [slots, heads, dk, dv].  With ``b`` (float32 rows
     [T, heads]): the gated delta rule, q and k made unit vectors (q times dk^-1/2), g = exp(-exp(a_log) softplus(a + dt_bias)),
     S <- g S, S += k (sigmoid(b) (v - S^T k))^T, o = S^T q.  With ``d_skip`` [heads]: dt = softplus(a + dt_bias),
-    S <- exp(-exp(a_log) dt) S + dt k v^T, o = S^T q + d_skip v.  ``carry`` (float32 scratch of ``gated_state_carry_floats``):
+    S <- exp(-exp(a_log) dt) S + dt k v^T, o = S^T q + d_skip v.  With ``decay`` [heads] (a, dt_bias and a_log are None): a fixed
+    decay, S <- decay S + k v^T, o = S^T q, of silu(q), silu(k), silu(v) where ``silu_in``.  ``carry`` (float32 scratch of ``gated_state_carry_floats``):
     runs are walked in pieces of ``piece`` rows, all pieces at once."""
     T = o.shape[0]
     delta = b is not None
-    _need(delta != (d_skip is not None), "gated_state: give b (the delta rule) or d_skip (the state-space recurrence)")
-    for t, n, c in ((q, "q", groups * dk), (k, "k", groups * dk), (v, "v", heads * dv), (a, "a", heads), (o, "o", heads * dv)) + (((b, "b", heads),) if delta else ()):
+    fixed = decay is not None
+    _need([delta, d_skip is not None, fixed].count(True) == 1,
+          "gated_state: give b (the delta rule), d_skip (the state-space recurrence) or decay (a fixed one)")
+    _need((a is None and dt_bias is None and a_log is None) if fixed else (a is not None and dt_bias is not None and a_log is not None),
+          "gated_state: a, dt_bias and a_log make the decays, unless they are fixed")
+    extra = (((b, "b", heads),) if delta else ()) + (() if fixed else ((a, "a", heads),))
+    for t, n, c in ((q, "q", groups * dk), (k, "k", groups * dk), (v, "v", heads * dv), (o, "o", heads * dv)) + extra:
         _f32rows(t, n, c)
         _need(t.shape[0] >= T, f"{n} has too few rows")
-    for t, n in ((dt_bias, "dt_bias"), (a_log, "a_log"), (d_skip, "d_skip")):
+    for t, n in ((dt_bias, "dt_bias"), (a_log, "a_log"), (d_skip, "d_skip"), (decay, "decay")):
         _f32(t, n, heads)
     _need(state.dtype == torch.float32 and state.is_contiguous() and state.is_cuda and tuple(state.shape[1:]) == (heads, dk, dv),
           "state must be float32 [slots, heads, dk, dv]")
     piece = int(piece or gated_state_piece(dk)) if carry is not None else 0
     _f32(carry, "carry")
-    _call("kvcm_gated_state", _ptr(q), q.stride(0), _ptr(k), k.stride(0), _ptr(v), v.stride(0), _ptr(a), a.stride(0), _ptr(b),
-          b.stride(0) if delta else 0, _ptr(dt_bias), _ptr(a_log), _ptr(d_skip), 1 if delta else 0, _ptr(o), o.stride(0), _ptr(state),
+    _call("kvcm_gated_state", _ptr(q), q.stride(0), _ptr(k), k.stride(0), _ptr(v), v.stride(0), _ptr(a),
+          0 if fixed else a.stride(0), _ptr(b), b.stride(0) if delta else 0, _ptr(dt_bias), _ptr(a_log), _ptr(d_skip), _ptr(decay),
+          1 if silu_in else 0, 1 if delta else 0, _ptr(o), o.stride(0), _ptr(state),
           _ptr(step.run_start), _ptr(step.seq_start), _ptr(step.state_slots), step.seqs, heads, groups, dk, dv, T, piece,
           int(step.max_run), _ptr(carry), carry.numel() if carry is not None else 0, _stream())
     return o

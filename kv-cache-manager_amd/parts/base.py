@@ -49,6 +49,7 @@ class ModelSpec:
     final_norm: PartSpec
     head: PartSpec
     max_position: int = 0
+    max_position_fixed: bool = False  # positions come from a table of max_position rows: no option lifts the limit
     keep_embedding: bool = False      # the embedding's output stays at hand for the layers (step.shared["embedding_output"])
 
 

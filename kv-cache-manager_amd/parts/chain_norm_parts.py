@@ -51,22 +51,30 @@ class ChainedRMSNorm(Norm):
     """out = x / sqrt(mean(x^2) + eps) * weight with every operation in 32-bit and one rounding at the end.
     ``forward`` also takes the previous sublayer's output that is still to be normed and added (``add``: what
     ``pending`` of the norm after that sublayer made), so that addition and norm are one launch.
-    params: size, eps; name: the checkpoint name of the weight (default prefix + "weight")."""
+    params: size, eps; offset: the weight is stored around it, the factor is offset + weight (default 0); factor: a constant
+    on the factor, for a norm whose result is added to the stream multiplied (default 1); name: the checkpoint name of the
+    weight (default prefix + "weight")."""
 
     capturable = True
     accepts_partial_sums = True      # ``add`` is taken as it comes (ops.NormedBranches)
 
     def param_specs(self):
         name = self.params.get("name", self.prefix + "weight")
-        return [ParamSpec("weight", ((name, (self.params["size"],)),), role="vector")]
+        return [ParamSpec("weight", ((name, (self.params["size"],)),), role="bias" if self.params.get("offset") else "vector")]
 
     def bind(self, tensors):
-        super().bind(f32_params(tensors))
+        w = f32_params(tensors)["weight"]
+        offset, factor = float(self.params.get("offset", 0.0)), float(self.params.get("factor", 1.0))
+        if offset != 0.0 or factor != 1.0:
+            w = ((w + offset) * factor).contiguous()
+        super().bind({"weight": w})
 
     def pending(self, value):
-        """A sublayer's output (a 32-bit tensor, ops.PartialSums, or a BranchPair) as what the stream's next norm adds:
-        x += n(value) * weight."""
+        """A sublayer's output (a 32-bit tensor, ops.PartialSums, a BranchPair, or ops.StreamTerms of one plain term) as what the
+        stream's next norm adds: x += n(value) * weight."""
         ops = self.ctx.ops
+        if isinstance(value, ops.StreamTerms):
+            value = value.only()
         if isinstance(value, BranchPair):
             return ops.NormedBranches(value.a, self.w["weight"], value.b, value.wa, value.wb, value.combine)
         return ops.NormedBranches(value, self.w["weight"])
@@ -132,21 +140,25 @@ class OutputNormResidual(Block):
 
 @EMBEDDINGS.register("scaled_token_embedding")
 class ScaledTokenEmbedding(Embedding):
-    """x = float(table[token]) * scale.  params: vocab_size, scale; name: the table's checkpoint name."""
+    """x = float(table[token]) * scale; with ``positions`` (a number of them) a learned vector per position is added as it is.
+    params: vocab_size, scale; name: the table's checkpoint name; positions; position_name: the checkpoint name of their table."""
 
     capturable = True
 
     def param_specs(self):
-        name = self.params.get("name", self.prefix + "weight")
-        return [ParamSpec("table", ((name, (self.params["vocab_size"], self.ctx.hidden_size)),), role="table")]
+        name, p, H = self.params.get("name", self.prefix + "weight"), self.params, self.ctx.hidden_size
+        specs = [ParamSpec("table", ((name, (p["vocab_size"], H)),), role="table")]
+        if p.get("positions"):
+            specs.append(ParamSpec("pos_table", ((p.get("position_name", self.prefix + "positions"), (p["positions"], H)),), role="table"))
+        return specs
 
     def forward(self, step, out):
-        self.ctx.ops.embed_scaled(step.tokens, self.w["table"], out, self.params.get("scale", 1.0))
+        self.ctx.ops.embed_scaled(step.tokens, self.w["table"], out, self.params.get("scale", 1.0),
+                                  positions=step.positions if "pos_table" in self.w else None, pos_table=self.w.get("pos_table"))
         return out
 
     def bytes_read(self, rows):
-        table = self.w["table"]
-        return rows * table.shape[1] * table.element_size()
+        return sum(rows * t.shape[1] * t.element_size() for t in self.w.values())
 
     def flops(self, rows, attended=0):
         return 0.0
@@ -155,9 +167,12 @@ class ScaledTokenEmbedding(Embedding):
 @FEED_FORWARDS.register("gated_mlp")
 class GatedFeedForward(JoinableEnds, FeedForward):
     """down(act(gate(h)) * up(h)), gate and up as one fused projection whose 32-bit sums go straight into the
-    activation (steps of few rows in bfloat16 with silu and without biases: in the product's own epilogue).  params: intermediate_size, activation ("relu" | "silu" | "gelu_tanh"); gate, up, down: the
+    activation (steps of few rows in bfloat16 with silu or "clamped" and without biases: in the product's own epilogue).
+    params: intermediate_size, activation ("relu" | "silu" | "gelu_tanh" | "gelu", or "clamped" with ``limit``: g * sigmoid(1.702 g) *
+    (u + 1) with g = min(gate, limit) and u = up held within +-limit); gate, up, down: the
     checkpoint names after the prefix (defaults "gate", "up", "down"); bias: all three projections have one (the tensor's
-    name + ".b").  The result is 32-bit: a norm reads it.  Offers its ends (JoinableEnds)."""
+    name + ".b"); partial_out: the last product may be handed on as un-added slices, to a norm that adds them (default: not).
+    The result is 32-bit: a norm reads it.  Offers its ends (JoinableEnds)."""
 
     capturable = True
 
@@ -184,7 +199,8 @@ class GatedFeedForward(JoinableEnds, FeedForward):
 
     def between(self, step, h, proj, out, row_gate=None):
         """``row_gate`` (32-bit rows, column 0): the output times sigmoid of it, one gate per row."""
-        self.ctx.ops.gated_act(proj, out, self.params.get("activation", "silu"), bias=self.w.get("b_gate_up"), row_gate=row_gate)
+        self.ctx.ops.gated_act(proj, out, self.params.get("activation", "silu"), bias=self.w.get("b_gate_up"), row_gate=row_gate,
+                               limit=self.params.get("limit", 0.0))
 
     def forward(self, step, h):
         I, ops = self.params["intermediate_size"], self.ctx.ops
@@ -194,12 +210,14 @@ class GatedFeedForward(JoinableEnds, FeedForward):
             return ops.BiasedOutput(linear32(self.ctx, step, act, self.w["w_down"], "gated_out", keep_partial=True), self.w["b_down"])
         act = step.ws("gated_act", (step.rows, I))
         kind = self.params.get("activation", "silu")
-        # few rows in bfloat16 with silu: the product that streams gate and up rows together and applies the activation
-        # in its epilogue, one launch (the activation is rounded once more on the way, within the result's own rounding)
-        if not (kind == "silu" and act.dtype == torch.bfloat16 and torch.is_tensor(h) and ops.gemm_swiglu(h, self.w["w_gate_up"], act)):
+        limit = self.params.get("limit", 0.0) if kind == "clamped" else 0.0
+        # few rows in bfloat16 with silu or its form with limits: the product that streams gate and up rows together and applies
+        # the activation in its epilogue, one launch (silu is rounded once more on the way, within the result's own rounding)
+        if not (kind in ("silu", "clamped") and act.dtype == torch.bfloat16 and torch.is_tensor(h)
+                and ops.gemm_swiglu(h, self.w["w_gate_up"], act, limit=limit)):
             gu = linear32(self.ctx, step, h, self.w["w_gate_up"], "gated_gate_up")
-            ops.gated_act(gu, act, kind)
-        return linear32(self.ctx, step, act, self.w["w_down"], "gated_out")
+            ops.gated_act(gu, act, kind, limit=limit)
+        return linear32(self.ctx, step, act, self.w["w_down"], "gated_out", keep_partial=bool(self.params.get("partial_out")))
 
 
 @FEED_FORWARDS.register("plain_mlp")

@@ -1,7 +1,7 @@
 """Mixers that carry a fixed-size 32-bit state per request instead of keys and values: the selective scan
 (with the short convolution in front of it), the generalized delta rule, a matrix memory with exponential gates, the gated
-delta rule and the state-space recurrence with one decay per head (the last two behind a short convolution).  Their states live in the
-cache manager's state slots; a request's portion that starts at position 0 starts from zero.  Every size,
+delta rule and the state-space recurrence with one decay per head (these two behind a short convolution), and lightning
+attention, whose decays are constants.  Their states live in the cache manager's state slots; a request's portion that starts at position 0 starts from zero.  Every size,
 constant and tensor name is a parameter.
 """
 import torch
@@ -191,15 +191,28 @@ class MatrixMemoryMixer(_StatefulMixer):
         return linear32(self.ctx, step, gated, w["w_o"], "memory_out", keep_partial=True)      # the stream's next norm adds the slices
 
 
-class _ConvStateMixer(EndsMixer):
-    """A short convolution (silu) over some of the projected channels, then a matrix state per head with one decay per head
-    and token (ops.gated_state).  Keeps per request: the state and the convolution's last taps-1 inputs, both 32-bit."""
+class _MatrixStateMixer(EndsMixer):
+    """A matrix state per head with one decay per head (ops.gated_state).  Keeps it per request, 32-bit."""
 
     capturable = True
 
     def state(self, name):
         storage, index, _ = self.caches[name]
         return storage.slots(index)
+
+    def carry(self, step, heads, dk, dv, delta):
+        """Scratch for walking long runs in pieces, sized for the engine's largest step; None for steps of short runs."""
+        ops = self.ctx.ops
+        if step.max_run < 4 * ops.gated_state_piece(dk):
+            return None
+        lim = step.limits
+        rows, seqs = max(step.rows, lim.max_tokens if lim else 0), max(step.seqs, lim.max_seqs if lim else 0)
+        return step.flat("gated_state_carry", ops.gated_state_carry_floats(rows, seqs, heads, dk, dv, delta))
+
+
+class _ConvStateMixer(_MatrixStateMixer):
+    """A short convolution (silu) over some of the projected channels, then a matrix state per head with one decay per head
+    and token.  Keeps per request: the state and the convolution's last taps-1 inputs, both 32-bit."""
 
     def needs(self, heads, dk, dv, taps, channels):
         needs = {"state": StateNeed((heads, dk, dv), torch.float32)}
@@ -218,15 +231,6 @@ class _ConvStateMixer(EndsMixer):
         if not single:
             ops.short_conv_state(x, state, step, taps)
         return mixed
-
-    def carry(self, step, heads, dk, dv, delta):
-        """Scratch for walking long runs in pieces, sized for the engine's largest step; None for steps of short runs."""
-        ops = self.ctx.ops
-        if step.max_run < 4 * ops.gated_state_piece(dk):
-            return None
-        lim = step.limits
-        rows, seqs = max(step.rows, lim.max_tokens if lim else 0), max(step.seqs, lim.max_seqs if lim else 0)
-        return step.flat("gated_state_carry", ops.gated_state_carry_floats(rows, seqs, heads, dk, dv, delta))
 
 
 @MIXERS.register("gated_delta")
@@ -342,3 +346,50 @@ class StateSpaceMixer(_ConvStateMixer):
                         self.state("state"), step, self.nh, self.groups, self.N, self.dv, d_skip=w["d_skip"],
                         carry=self.carry(step, self.nh, self.N, self.dv, False))
         ops.group_norm_gate(y, proj, w["norm"], out, self.norm_groups, inner // self.norm_groups, p["eps"])
+
+
+@MIXERS.register("lightning_attention")
+class LightningAttention(_MatrixStateMixer):
+    """Linear attention with a constant decay per head.  q = silu(W_q h), k = silu(W_k h) (heads of dim), v = silu(W_v h) (heads
+    of vdim); S <- decay_h S + k v^T, o = S^T q; all heads' o side by side are divided by their root mean square together, times
+    a weight, times sigmoid(W_g h), then the output projection.
+    params: heads, dim, vdim, decay (a number per head), eps, out_factor (on the output, default 1).
+    Tensors under the prefix: q, k, v, g, norm, o."""
+
+    ends_name = "lightning"
+
+    def __init__(self, params, prefix, ctx):
+        super().__init__(params, prefix, ctx)
+        self.nh, self.d, self.dv = params["heads"], params["dim"], params["vdim"]
+        if len(params["decay"]) != self.nh:
+            raise ValueError(f"lightning_attention {prefix!r}: {len(params['decay'])} decays for {self.nh} heads")
+
+    def in_sources(self):
+        H, pre, nk, nv = self.ctx.hidden_size, self.prefix, self.nh * self.d, self.nh * self.dv
+        return tuple((pre + n, (c, H)) for n, c in (("q", nk), ("k", nk), ("v", nv), ("g", nv)))
+
+    def out_source(self):
+        return (self.prefix + "o", (self.ctx.hidden_size, self.nh * self.dv))
+
+    def own_specs(self):
+        return [ParamSpec("norm", ((self.prefix + "norm", (self.nh * self.dv,)),), role="vector")]
+
+    def bind(self, tensors):
+        super().bind(tensors)
+        self.w["norm"] = (self.w["norm"] * float(self.params.get("out_factor", 1.0))).contiguous()
+        self.w["decay"] = torch.tensor(self.params["decay"], dtype=torch.float32, device=self.w["norm"].device)
+
+    def cache_needs(self):
+        return {"state": StateNeed((self.nh, self.d, self.dv), torch.float32)}
+
+    def flops(self, rows, attended=0):
+        return super().flops(rows) + rows * self.nh * 5.0 * self.d * self.dv
+
+    def between(self, step, h, proj, out):
+        ops, w = self.ctx.ops, self.w
+        nh, d, dv = self.nh, self.d, self.dv
+        q, k, v, g = (proj[:, at:] for at in (0, nh * d, 2 * nh * d, 2 * nh * d + nh * dv))
+        o = step.ws("lightning_o", (step.rows, nh * dv), torch.float32)
+        ops.gated_state(q, k, v, None, None, None, o, self.state("state"), step, nh, nh, d, dv, decay=w["decay"], silu_in=True,
+                        carry=self.carry(step, nh, d, dv, False))
+        ops.group_norm_gate(o, g, w["norm"], out, 1, nh * dv, self.params["eps"], after=True)

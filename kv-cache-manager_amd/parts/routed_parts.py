@@ -24,16 +24,19 @@ class RoutedExperts(JoinableEnds, FeedForward):
       "softmax" (default)  router logits z = W_router h in 32-bit, scores s = softmax(z) over all experts; the ``top``
                            experts with the largest scores, weighted by their scores as they are (not renormalized)
       "softmax_chosen"     the ``top`` experts with the largest logits, weighted by the softmax over those logits alone
+      "sigmoid"            scores s = sigmoid(z), each of its own logit; the ``top`` largest, weighted by their scores as they are
       "table"              an integer table [vocabulary, top] names the experts of every token id; each weighs 1 / top
     What an expert computes (``activation``):
       "relu2" (default)    W_down act(W_up h), act = the square of relu
+      "gelu"               W_down act(W_up h), act = the exact gelu (by the error function)
       "silu_gated"         W_down (silu(W_gate h) * (W_up h))
+    ``weigh``: "output" (default): the row gets the sum of weight * expert(h); "input": the sum of expert(weight * h).
     Experts have no biases.  ``shared``: a PartSpec of a feed-forward that runs for every row and is added (default none).
     ``shared_gate``: the shared feed-forward's output is multiplied by sigmoid(W_sg h), one number per row (the tensor's name
     after the prefix; default none).  ``route_factor``: a constant on the experts' weights (default 1).
     Offers its ends (JoinableEnds): the router's product, the gate's and the shared feed-forward's first at one end, the shared
     feed-forward's last at the other; the experts' sum is the further output.  With ``shared_gate`` it runs that way on its own too.
-    params: experts, top, ff, routing, activation, shared, shared_gate, route_factor, vocab_size (rows of the table; default: as stored); router / table (the checkpoint name after the prefix, defaults
+    params: experts, top, ff, routing, activation, weigh, shared, shared_gate, route_factor, vocab_size (rows of the table; default: as stored); router / table (the checkpoint name after the prefix, defaults
     "router", "table"); expert (a pattern for an expert's prefix, default "e{}."), gate, up, down (names after it).
     The result is 32-bit."""
 
@@ -45,10 +48,12 @@ class RoutedExperts(JoinableEnds, FeedForward):
     def __init__(self, params, prefix, ctx):
         super().__init__(params, prefix, ctx)
         self.routing, self.activation = params.get("routing", "softmax"), params.get("activation", "relu2")
-        if self.routing not in ("softmax", "softmax_chosen", "table"):
-            raise ValueError(f"routed_experts {prefix!r}: routing {self.routing!r} is not supported (softmax | softmax_chosen | table)")
-        if self.activation not in ("relu2", "silu_gated"):
-            raise ValueError(f"routed_experts {prefix!r}: activation {self.activation!r} is not supported (relu2 | silu_gated)")
+        if self.routing not in ("softmax", "softmax_chosen", "sigmoid", "table"):
+            raise ValueError(f"routed_experts {prefix!r}: routing {self.routing!r} is not supported (softmax | softmax_chosen | sigmoid | table)")
+        if self.activation not in ("relu2", "gelu", "silu_gated"):
+            raise ValueError(f"routed_experts {prefix!r}: activation {self.activation!r} is not supported (relu2 | gelu | silu_gated)")
+        if params.get("weigh", "output") not in ("output", "input"):
+            raise ValueError(f"routed_experts {prefix!r}: weigh {params['weigh']!r} is not supported (output | input)")
         self.gated = self.activation == "silu_gated"
         sh = params.get("shared")
         self.by_ends = bool(params.get("joined") or params.get("shared_gate"))
@@ -174,10 +179,11 @@ class RoutedExperts(JoinableEnds, FeedForward):
         else:
             if logits is None:
                 logits = linear32(self.ctx, step, h, w["w_router"], "routed_logits", keep_partial=True)      # the route adds the slices
-            ops.moe_route(logits, E, top, chosen, weight, rows=T, over_chosen=self.routing == "softmax_chosen",
+            ops.moe_route(logits, E, top, chosen, weight, rows=T, over_chosen=self.routing == "softmax_chosen", sigmoid=self.routing == "sigmoid",
                           factor=p.get("route_factor", 1.0))
         add = self.shared.forward(step, h) if self.shared is not None and not self.by_ends else None      # 32-bit [T, H]: the experts' sum starts from it
         H = self.ctx.hidden_size
+        how = dict(gated=self.gated, add=add, weigh_input=p.get("weigh") == "input", **({} if self.gated else {"activation": self.activation}))
         act = step.ws("routed_act", (T, top * F)).view(T * top, F)
         out = step.ws("routed_out", (T, H), torch.float32)
         if T >= self.GROUPED_MIN_ROWS and ops.moe_grouped_supported(H, F, E, act.dtype) and h.stride(0) % 8 == 0:
@@ -185,5 +191,5 @@ class RoutedExperts(JoinableEnds, FeedForward):
             order = step.ws("routed_order", (T, top), torch.int32)
             tiles = step.flat("routed_tiles", ops.moe_grouped_tiles(max(T, step.limits.max_tokens if step.limits else T) * top, E), torch.int32)
             y = step.ws("routed_y", (T, top * H), torch.float32).view(T * top, H)
-            return ops.moe_grouped(h, w["w_up"], w["w_down"], chosen, weight, order, tiles, act, y, out, gated=self.gated, add=add)
-        return ops.moe_rows(h, w["w_up"], w["w_down"], chosen, weight, act, out, gated=self.gated, add=add)
+            return ops.moe_grouped(h, w["w_up"], w["w_down"], chosen, weight, order, tiles, act, y, out, **how)
+        return ops.moe_rows(h, w["w_up"], w["w_down"], chosen, weight, act, out, **how)
