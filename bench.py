@@ -285,6 +285,28 @@ def vugotar_config(width, layers, vocab=32000):
     return VugotarConfig.from_dict({"architecture": "Vugotar", "vocab": vocab, "width": width, "norm": {"eps": 1e-6}, "layers": listed})
 
 
+# Zalunex at a width: (experts, experts a row, limit of the dense feed-forward's gate); the other sizes are DESIGN_SIZES'
+ZALUNEX_SIZES = {2048: (8, 2, 7.0), 4096: (8, 2, 7.0)}
+
+
+def zalunex_config(width, layers, vocab=32000):
+    """A Zalunex configuration at a width of DESIGN_SIZES: every layer has window attention (the other designs' heads and window)
+    beside lightning attention of as many heads, keys and values of the attention's size, decays spread from 0.9 to 0.999; the
+    first and third of four have a dense feed-forward, the others ``experts`` gelu experts of which a row uses ``top`` (together
+    as wide as the dense feed-forward)."""
+    from kvcm_amd.config.zalunex_config import ZalunexConfig
+    nh, nkv, hd, ff, window = DESIGN_SIZES[width][:5]
+    experts, top, limit = ZALUNEX_SIZES[width]
+    moe = {"kind": "moe", "expert": {"ff": ff // top}, "router": {"experts": experts, "top": top}}
+    dense = {"kind": "dense", "ff": ff, "limit": limit}
+    left = {"heads": nh, "kv_heads": nkv, "dim": hd, "vdim": hd, "scale": hd ** -0.5, "mask": {"size": window}}
+    right = {"heads": nh, "dim": hd, "vdim": hd, "decay": [1.0 - 10.0 ** (-1.0 - 2.0 * h / (nh - 1)) for h in range(nh)]}
+    parallel = {"left": left, "right": right, "left_scale": 1.1, "right_scale": 0.6}
+    listed = [{"type": "parallel", "mixer": parallel, "mlp": dense if i % 2 == 0 else moe} for i in range(layers)]
+    return ZalunexConfig.from_dict({"architecture": "Zalunex", "vocab": vocab, "width": width, "max_positions": 16384, "norm": {"eps": 1e-6},
+                                    "residual_mult": 0.8, "logit_softcap": 30.0, "layers": listed})
+
+
 def design_main(args):
     import torch
     from kvcm_amd.config.engine_config import EngineConfig
@@ -300,7 +322,8 @@ def design_main(args):
     record = {"metric": "prefill and decode tok/s of the %s decoder beside the %s at equal sizes"
                         % (first.capitalize(), {"kasuvik": "Llama decoder", "furapel": "Kasuvik and Llama decoders",
                                                  "fisesun": "Furapel and Llama decoders", "betirax": "Fisesun and Llama decoders",
-                                                 "vugotar": "Kasuvik, Betirax and Llama decoders"}[first]), "dtype": key,
+                                                 "vugotar": "Kasuvik, Betirax and Llama decoders",
+                                                 "zalunex": "Vugotar, Kasuvik and Llama decoders"}[first]), "dtype": key,
               "data": "synthetic", "layers": layers, "prefill_tokens": T, "prompt_len": args.prompt_len, "steps": steps, "sizes": {}}
     for width in [int(w) for w in args.design_sizes.split(",")]:
         if width not in DESIGN_SIZES:
@@ -317,10 +340,14 @@ def design_main(args):
         elif first == "vugotar":
             designs = {"vugotar": vugotar_config(width, layers), "kasuvik": designs["kasuvik"], "betirax": betirax_config(width, layers),
                        "llama": designs["llama"]}
+        elif first == "zalunex":
+            designs = {"zalunex": zalunex_config(width, layers), "vugotar": vugotar_config(width, layers), "kasuvik": designs["kasuvik"],
+                       "llama": designs["llama"]}
         if args.design_alone:
             designs = {first: designs[first]}
         for name, cfg in designs.items():
-            arch = {"kasuvik": "Kasuvik", "furapel": "Furapel", "fisesun": "Fisesun", "betirax": "Betirax", "vugotar": "Vugotar", "llama": "LlamaForCausalLM"}[name]
+            arch = {"kasuvik": "Kasuvik", "furapel": "Furapel", "fisesun": "Fisesun", "betirax": "Betirax", "vugotar": "Vugotar", "zalunex": "Zalunex",
+                    "llama": "LlamaForCausalLM"}[name]
             tensors = random_tensors(arch, cfg, seed=0, dtype=dt, device="cuda:0")
             ec = EngineConfig(block_size=16, max_seq_len=limit, num_blocks=8 * limit // 16, max_num_seqs=8,
                               max_batched_tokens=max(4096, T + 64), dtype=args.dtype, max_logit_rows=64, beyond_max_position=True)
@@ -373,12 +400,13 @@ def main():
                     help="run nothing but the 2,048-token prefill (for a profiler); prints its record alone")
     ap.add_argument("--prefill-tokens", type=int, default=2048,
                     help="tokens of the prefill measurement (2,048 in the record; other lengths for sweeps)")
-    ap.add_argument("--design", default="llama", choices=["llama", "kasuvik", "furapel", "fisesun", "betirax", "vugotar"],
+    ap.add_argument("--design", default="llama", choices=["llama", "kasuvik", "furapel", "fisesun", "betirax", "vugotar", "zalunex"],
                     help="llama: the workload above (the default); kasuvik: prefill and decode of the Kasuvik decoder beside the "
                          "Llama decoder at equal sizes; furapel: the same for the Furapel decoder beside both; "
                          "fisesun: the same for the Fisesun decoder beside the Furapel and the Llama decoder; "
                          "betirax: the same for the Betirax decoder beside the Fisesun and the Llama decoder; "
-                         "vugotar: the same for the Vugotar decoder beside the Kasuvik, the Betirax and the Llama decoder "
+                         "vugotar: the same for the Vugotar decoder beside the Kasuvik, the Betirax and the Llama decoder; "
+                         "zalunex: the same for the Zalunex decoder beside the Vugotar, the Kasuvik and the Llama decoder "
                          "(--design-sizes, --layers, --prefill-tokens, --prompt-len, --steps)")
     ap.add_argument("--design-sizes", default="2048,4096", help="widths of the --design comparison (2048, 4096)")
     ap.add_argument("--design-alone", action="store_true", help="run the --design itself only, not the designs beside it (for a profiler)")

@@ -54,6 +54,19 @@ __device__ __forceinline__ float ff_activation(int act, float z) {
   return z / (1.0f + expf(-z));
 }
 
+// The exact gelu for a result stored as T.  For a bfloat16 result the error function is the five-term approximation of
+// Abramowitz and Stegun's handbook (formula 7.1.26, absolute error up to 1.5e-7) in its complementary form, with the hardware's
+// exp2 and reciprocal: erfc(x) = (a1 t + .. + a5 t^5) exp(-x^2), t = 1 / (1 + p x), x >= 0.
+template <class T> __device__ __forceinline__ float gelu_exact(float z);
+template <> __device__ __forceinline__ float gelu_exact<float>(float z) { return ff_activation(3, z); }
+template <> __device__ __forceinline__ float gelu_exact<bf16_t>(float z) {
+  const float x = fabsf(z) * 0.70710678118654752f;
+  const float t = __builtin_amdgcn_rcpf(fmaf(0.3275911f, x, 1.0f));
+  const float poly = t * fmaf(t, fmaf(t, fmaf(t, fmaf(t, 1.061405429f, -1.453152027f), 1.421413741f), -0.284496736f), 0.254829592f);
+  const float half_erfc = 0.5f * poly * __builtin_amdgcn_exp2f(-1.44269504088896341f * x * x);      // the distribution's tail beyond |z|
+  return z * (z < 0.f ? half_erfc : 1.0f - half_erfc);
+}
+
 // A gate with limits: g = min(gate, limit), u = up held within [-limit, limit], g / (1 + exp(-1.702 g)) * (u + 1).
 constexpr float kClampedGateSlope = 1.702f;
 template <class T> __device__ __forceinline__ float clamped_gate(float gate, float up, float limit) {

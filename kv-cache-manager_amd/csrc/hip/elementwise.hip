@@ -427,6 +427,17 @@ __global__ void add_residual_kernel(float* __restrict__ x, const T* __restrict__
 
 
 // ---------------------------------------------------------------- embedding with a factor
+// four stored values at a multiple-of-four place of a row
+__device__ __forceinline__ void load4_f(const float* p, float* f) {
+  const float4 v = *reinterpret_cast<const float4*>(p);
+  f[0] = v.x; f[1] = v.y; f[2] = v.z; f[3] = v.w;
+}
+__device__ __forceinline__ void load4_f(const bf16_t* p, float* f) {
+  const uint2 v = *reinterpret_cast<const uint2*>(p);
+  f[0] = bf16_bits_to_float(v.x & 0xffffu); f[1] = bf16_bits_to_float(v.x >> 16);
+  f[2] = bf16_bits_to_float(v.y & 0xffffu); f[3] = bf16_bits_to_float(v.y >> 16);
+}
+
 template <class TW>
 __global__ void embed_scaled_kernel(const int* __restrict__ ids, const TW* __restrict__ table, float* __restrict__ x,
                                     int H, int V, float factor, const int* __restrict__ positions, const TW* __restrict__ pos_table,
@@ -439,6 +450,22 @@ __global__ void embed_scaled_kernel(const int* __restrict__ ids, const TW* __res
     return;
   }
   const TW* src = table + size_t(id) * H;
+  if (H % 4 == 0) {      // four values a load and a store
+    const int pp = pos_table ? positions[t] : -1;
+    const bool here = pp >= 0 && pp < P;
+    const TW* at = here ? pos_table + size_t(pp) * H : src;
+    const float add = here ? 1.f : 0.f;
+    for (int i = threadIdx.x * 4; i < H; i += blockDim.x * 4) {
+      float a[4], b[4];
+      load4_f(src + i, a);
+      load4_f(at + i, b);
+      float4 v;
+      v.x = fmaf(a[0], factor, add * b[0]); v.y = fmaf(a[1], factor, add * b[1]);
+      v.z = fmaf(a[2], factor, add * b[2]); v.w = fmaf(a[3], factor, add * b[3]);
+      *reinterpret_cast<float4*>(dst + i) = v;
+    }
+    return;
+  }
   const int p = pos_table ? positions[t] : -1;      // a learned vector per position, unscaled (no position beyond the table gets here)
   if (p >= 0 && p < P) {
     const TW* at = pos_table + size_t(p) * H;

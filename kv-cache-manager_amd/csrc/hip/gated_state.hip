@@ -123,7 +123,7 @@ __global__ void __launch_bounds__(256) gated_state_kernel(StateArgs A) {
 #pragma unroll
     for (int n = 0; n < PF; ++n) {
       const int e = threadIdx.x + n * 256;
-      if (e < TILE * V) tile[e / V][e % V] = !DELTA && A.silu_in ? silu<float>(pf[n]) : pf[n];      // (silu(0) = 0: what was masked stays 0)
+      if (e < TILE * V) tile[e / V][e % V] = !DELTA && A.silu_in ? silu<bf16_t>(pf[n]) : pf[n];      // (silu(0) = 0: what was masked stays 0)
     }
     if (threadIdx.x < TILE) {
       const float dt = softplus32(sa + dtb);

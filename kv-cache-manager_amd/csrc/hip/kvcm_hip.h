@@ -247,6 +247,11 @@ int kvcm_gated_state(const float* q, int ldq, const float* k, int ldk, const flo
                      int ldb, const float* dt_bias, const float* a_log, const float* d_skip, const float* decay, int silu_in, int delta, float* o, int ldo, float* state,
                      const int* run_start, const int* seq_start, const int* state_slots, int S, int heads, int groups, int dk, int dv,
                      int T, int piece, int max_run, float* carry, long long carry_floats, hipStream_t s);
+// (lightning.hip) a matrix state per head with a constant decay, runs of rows in matrix form
+long long kvcm_lightning_carry_floats(int rows, int S, int heads, int dk, int dv, int piece);
+int kvcm_lightning(const float* q, int ldq, const float* k, int ldk, const float* v, int ldv, const float* powers, int silu_in, float* o,
+                   int ldo, float* state, const int* run_start, const int* seq_start, const int* state_slots, int S, int heads, int dk,
+                   int dv, int T, int piece, int max_run, float* carry, long long carry_floats, hipStream_t s);
 // (mlstm.hip) a matrix memory with exponential gates, walked token by token
 int kvcm_mlstm_scan(const float* q, int ldq, const float* k, int ldk, const float* v, int ldv, const float* ig, int ldi,
                     const float* fg, int ldf, const float* i_bias, const float* f_bias, float cap, float q_scale, float* coef,

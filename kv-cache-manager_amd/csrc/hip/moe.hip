@@ -186,7 +186,7 @@ __global__ void __launch_bounds__(256)
   if (lane == 0)
     for (int c = 0; c < cols; ++c) {
       const float y = g * z[c], r = fmaxf(y, 0.f);
-      store_f(act + size_t(item) * F + c0 + c, kind == 2 ? ff_activation(3, y) : r * r);
+      store_f(act + size_t(item) * F + c0 + c, kind == 2 ? gelu_exact<T>(y) : r * r);
     }
 }
 
@@ -199,7 +199,14 @@ __global__ void __launch_bounds__(256)
   extern __shared__ __attribute__((aligned(16))) float xs[];      // [top][F4], F4: F rounded up to 4
   const int row = blockIdx.x;
   const int F4 = (F + 3) & ~3;
-  for (int k = threadIdx.x; k < top * F; k += 256) xs[(k / F) * F4 + k % F] = load_f(act + size_t(row) * top * F + k);
+  if (F % Piece<T>::N == 0) {      // 16 bytes a load
+    constexpr int N = Piece<T>::N;
+    for (int s = 0; s < top; ++s)
+      for (int k = threadIdx.x * N; k < F; k += 256 * N) unpack16(act + (size_t(row) * top + s) * F + k, xs + s * F4 + k);
+  } else {
+    for (int s = 0; s < top; ++s)
+      for (int k = threadIdx.x; k < F; k += 256) xs[s * F4 + k] = load_f(act + (size_t(row) * top + s) * F + k);
+  }
   __syncthreads();
   const int wave = threadIdx.x / kWave, lane = threadIdx.x % kWave;
   const bool vec = F % Piece<T>::N == 0;

@@ -181,14 +181,41 @@ __global__ void __launch_bounds__(256)
     }
     return;
   }
+  if constexpr (MODE == kUp || MODE == kUpGelu) {
+    // activations without a gate, in grouped order: a wave's 64 x 64 of them pass through LDS as well and are written in whole
+    // 128-byte stretches of a row, 16 bytes a lane (N is a multiple of 8: a piece lies inside or outside)
+    constexpr int kPitch = 72;
+    static_assert(4 * 64 * kPitch * sizeof(uint16_t) <= sizeof(staged), "the activations of a tile must fit the operands' space");
+    uint16_t* mine = &staged[0][0][0] + wave * 64 * kPitch;
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int ml = i * 16 + (lane / 16) * 4 + r;
+        const float g = weight ? weight[pair_of[wm * 64 + ml]] : 1.f;      // a factor on what the expert reads
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+          const float v = g * acc[i][j][r], z = fmaxf(v, 0.f);
+          mine[ml * kPitch + j * 16 + lane % 16] = float_to_bf16_bits(MODE == kUpGelu ? gelu_exact<bf16_t>(v) : z * z);
+        }
+      }
+    __syncthreads();
+#pragma unroll
+    for (int it = 0; it < 8; ++it) {
+      const int idx = it * kWave + lane, ml = idx / 8, c8 = (idx % 8) * 8, c = n0 + wn * 64 + c8;
+      if (wm * 64 + ml >= rows || c >= N) continue;
+      *reinterpret_cast<uint4*>(static_cast<uint16_t*>(out) + static_cast<long long>(p0 + wm * 64 + ml) * N + c) =
+          *reinterpret_cast<const uint4*>(mine + ml * kPitch + c8);
+    }
+    return;
+  }
 #pragma unroll
   for (int i = 0; i < 4; ++i)
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
       const int m = wm * 64 + i * 16 + (lane / 16) * 4 + r;
       if (m >= rows) continue;
-      const int pair = pair_of[m];
-      const float g = weight ? weight[pair] : 1.f;      // (the down form returned above: here a factor on what the expert reads)
+      const float g = weight ? weight[pair_of[m]] : 1.f;
       if constexpr (MODE == kUpGated) {
 #pragma unroll
         for (int j = 0; j < 4; j += 2) {      // tile j: sixteen gate columns, tile j + 1: the same sixteen up columns
@@ -197,15 +224,6 @@ __global__ void __launch_bounds__(256)
           const int col = (n0 + wn * 64 + j * 16) / 2 + lane % 16;
           static_cast<uint16_t*>(out)[static_cast<long long>(p0 + m) * (N / 2) + col] =
               float_to_bf16_bits(silu<bf16_t>(g * acc[i][j][r]) * (g * acc[i][j + 1][r]));
-        }
-      } else {
-#pragma unroll
-        for (int j = 0; j < 4; ++j) {
-          const int c = n0 + wn * 64 + j * 16 + lane % 16;
-          if (c >= N) continue;
-          const float v = g * acc[i][j][r], z = fmaxf(v, 0.f);
-          static_cast<uint16_t*>(out)[static_cast<long long>(p0 + m) * N + c] =
-              float_to_bf16_bits(MODE == kUpGelu ? ff_activation(3, v) : z * z);
         }
       }
     }

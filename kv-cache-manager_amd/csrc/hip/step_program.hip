@@ -127,6 +127,7 @@ const Entry kEntries[] = {
     KVCM_ENTRY(kvcm_stream_terms),
     KVCM_ENTRY(kvcm_group_norm_gate),
     KVCM_ENTRY(kvcm_gated_state),
+    KVCM_ENTRY(kvcm_lightning),
 };
 #undef KVCM_ENTRY
 

@@ -133,13 +133,13 @@ __global__ void __launch_bounds__(kTermThreads)
   }
 }
 
-// one workgroup per (row, group); groups of up to 4,096 values are read once and kept in registers
-template <class TO>
+// one workgroup per (row, group); groups of up to 256 HELD values are read once, all loads on their way together, and kept in
+// registers
+template <class TO, int HELD>
 __global__ void __launch_bounds__(kTermThreads)
     group_norm_gate_kernel(const float* __restrict__ y, int ldy, const float* __restrict__ z, int ldz, const float* __restrict__ w,
                            TO* __restrict__ out, int ldo, int size, float eps, int after) {
   __shared__ float scratch[kTermThreads / kWave];
-  constexpr int kHeld = 16;
   const int row = blockIdx.x, c0 = blockIdx.y * size;
   const float* yr = y + size_t(row) * ldy + c0;
   const float* zr = z + size_t(row) * ldz + c0;
@@ -149,20 +149,27 @@ __global__ void __launch_bounds__(kTermThreads)
     const float g = zr[i];
     return yr[i] * (g / (1.0f + expf(-g)));
   };
-  if (size <= kHeld * kTermThreads) {
-    float v[kHeld], gate[kHeld], ss = 0.f;
+  if (size <= HELD * kTermThreads) {
+    float v[HELD], z4[HELD], ss = 0.f;
 #pragma unroll
-    for (int j = 0; j < kHeld; ++j) {
+    for (int j = 0; j < HELD; ++j) {
+      const int i = threadIdx.x + j * kTermThreads, ic = i < size ? i : 0;
+      v[j] = yr[ic];
+      z4[j] = zr[ic];
+    }
+#pragma unroll
+    for (int j = 0; j < HELD; ++j) {
       const int i = threadIdx.x + j * kTermThreads;
-      v[j] = i < size ? value(i) : 0.f;
-      gate[j] = (after && i < size) ? 1.0f / (1.0f + expf(-zr[i])) : 1.f;
+      const float sg = 1.0f / (1.0f + expf(-z4[j]));
+      v[j] = i < size ? (after ? v[j] : v[j] * (z4[j] * sg)) : 0.f;
+      z4[j] = after ? sg : 1.f;
       ss = fmaf(v[j], v[j], ss);
     }
     const float inv = 1.0f / sqrtf(terms_block_sum(ss, scratch) / float(size) + eps);
 #pragma unroll
-    for (int j = 0; j < kHeld; ++j) {
+    for (int j = 0; j < HELD; ++j) {
       const int i = threadIdx.x + j * kTermThreads;
-      if (i < size) store_f(o + i, v[j] * inv * w[c0 + i] * gate[j]);
+      if (i < size) store_f(o + i, v[j] * inv * w[c0 + i] * z4[j]);
     }
     return;
   }
@@ -221,11 +228,17 @@ int kvcm_group_norm_gate(const float* y, int ldy, const float* z, int ldz, const
   KVCM_REQUIRE(T > 0 && groups > 0 && size > 0 && y && z && w && out, "group_norm_gate: bad sizes T=%d groups=%d size=%d", T, groups, size);
   KVCM_REQUIRE(groups <= 65535 && ldy >= groups * size && ldz >= groups * size && ldo >= groups * size, "group_norm_gate: row strides too small");
   const dim3 grid(T, groups);
-  if (out_dtype == kF32)
-    group_norm_gate_kernel<float><<<grid, kTermThreads, 0, s>>>(y, ldy, z, ldz, w, static_cast<float*>(out), ldo, size, eps, after);
-  else if (out_dtype == kBF16)
-    group_norm_gate_kernel<bf16_t><<<grid, kTermThreads, 0, s>>>(y, ldy, z, ldz, w, static_cast<bf16_t*>(out), ldo, size, eps, after);
+#define KVCM_GROUP_NORM(TO)                                                                                                        \
+  {                                                                                                                                \
+    TO* oo = static_cast<TO*>(out);                                                                                                \
+    if (size <= 1024) group_norm_gate_kernel<TO, 4><<<grid, kTermThreads, 0, s>>>(y, ldy, z, ldz, w, oo, ldo, size, eps, after);    \
+    else if (size <= 2048) group_norm_gate_kernel<TO, 8><<<grid, kTermThreads, 0, s>>>(y, ldy, z, ldz, w, oo, ldo, size, eps, after); \
+    else group_norm_gate_kernel<TO, 16><<<grid, kTermThreads, 0, s>>>(y, ldy, z, ldz, w, oo, ldo, size, eps, after);                \
+  }
+  if (out_dtype == kF32) KVCM_GROUP_NORM(float)
+  else if (out_dtype == kBF16) KVCM_GROUP_NORM(bf16_t)
   else KVCM_REQUIRE(false, "group_norm_gate: unknown output dtype %d", out_dtype);
+#undef KVCM_GROUP_NORM
   return launch_status("group_norm_gate");
 }
 

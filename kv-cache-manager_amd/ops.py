@@ -125,6 +125,9 @@ def _declare(lib):
     fn("kvcm_stream_terms", vp, vp, i, f, vp, i, f, vp, i, f, C.c_longlong, vp, vp, vp, vp, vp, i, i, i, f, vp)
     fn("kvcm_group_norm_gate", vp, i, vp, i, vp, vp, i, i, i, i, i, f, i, vp)
     fn("kvcm_gated_state", vp, i, vp, i, vp, i, vp, i, vp, i, vp, vp, vp, vp, i, i, vp, i, vp, vp, vp, vp, i, i, i, i, i, i, i, i, vp, C.c_longlong, vp)
+    fn("kvcm_lightning", vp, i, vp, i, vp, i, vp, i, vp, i, vp, vp, vp, vp, i, i, i, i, i, i, i, vp, C.c_longlong, vp)
+    lib.kvcm_lightning_carry_floats.restype = C.c_longlong
+    lib.kvcm_lightning_carry_floats.argtypes = [i] * 6
     lib.kvcm_gated_state_carry_floats.restype = C.c_longlong
     lib.kvcm_gated_state_carry_floats.argtypes = [i] * 7
     fn("kvcm_scan_prepare", vp, i, vp, vp, i, i, i, vp)
@@ -1874,4 +1877,46 @@ def gated_state(q, k, v, a, dt_bias, a_log, o, state, step, heads, groups, dk, d
           1 if silu_in else 0, 1 if delta else 0, _ptr(o), o.stride(0), _ptr(state),
           _ptr(step.run_start), _ptr(step.seq_start), _ptr(step.state_slots), step.seqs, heads, groups, dk, dv, T, piece,
           int(step.max_run), _ptr(carry), carry.numel() if carry is not None else 0, _stream())
+    return o
+
+
+LIGHTNING_ROWS = 64          # rows of a chunk of ``lightning``
+LIGHTNING_MIN_RUN = 16       # rows of a run from which its matrix form is worth it; shorter ones are walked (``gated_state``)
+
+
+def lightning_piece(dk):
+    """Rows of a piece when long runs are walked in pieces."""
+    return 128 if dk <= 64 else 256
+
+
+def lightning_powers(decay, piece, device):
+    """[heads, 66] float32 for ``lightning``: decay^0 .. decay^64 and decay^piece of every head, made in double precision."""
+    d = torch.tensor([float(x) for x in decay], dtype=torch.float64)
+    exponents = torch.tensor(list(range(LIGHTNING_ROWS + 1)) + [piece], dtype=torch.float64)
+    return torch.pow(d[:, None], exponents[None, :]).to(torch.float32).contiguous().to(device)
+
+
+def lightning_carry_floats(rows, seqs, heads, dk, dv, piece=None):
+    """32-bit values of scratch that ``lightning`` needs to walk a step of this shape in pieces."""
+    return int(lib().kvcm_lightning_carry_floats(rows, seqs, heads, dk, dv, piece or lightning_piece(dk)))
+
+
+def lightning(q, k, v, powers, o, state, step, heads, dk, dv, silu_in=False, carry=None, piece=None):
+    """A matrix state per head with a constant decay over the step's runs, in matrix form (csrc/hip/lightning.hip):
+    S <- decay S + k v^T, o = S^T q, of silu(q), silu(k), silu(v) where ``silu_in``.  q, k [T, heads*dk], v [T, heads*dv]:
+    float32 rows; ``powers``: ``lightning_powers`` of the decays and ``piece`` (default ``lightning_piece``); state [slots,
+    heads, dk, dv].  ``carry`` (float32 scratch of ``lightning_carry_floats``): needed where a run is longer than a piece."""
+    T = o.shape[0]
+    piece = int(piece or lightning_piece(dk))
+    for t, n, c in ((q, "q", heads * dk), (k, "k", heads * dk), (v, "v", heads * dv), (o, "o", heads * dv)):
+        _f32rows(t, n, c)
+        _need(t.shape[0] >= T, f"{n} has too few rows")
+    _f32(powers, "powers", heads * (LIGHTNING_ROWS + 2))
+    _need(state.dtype == torch.float32 and state.is_contiguous() and state.is_cuda and tuple(state.shape[1:]) == (heads, dk, dv),
+          "state must be float32 [slots, heads, dk, dv]")
+    _f32(carry, "carry")
+    _need(carry is not None or step.max_run <= piece, "lightning: runs longer than a piece need the scratch for pieces")
+    _call("kvcm_lightning", _ptr(q), q.stride(0), _ptr(k), k.stride(0), _ptr(v), v.stride(0), _ptr(powers), 1 if silu_in else 0, _ptr(o),
+          o.stride(0), _ptr(state), _ptr(step.run_start), _ptr(step.seq_start), _ptr(step.state_slots), step.seqs, heads, dk, dv, T,
+          piece if carry is not None else 0, int(step.max_run), _ptr(carry), carry.numel() if carry is not None else 0, _stream())
     return o

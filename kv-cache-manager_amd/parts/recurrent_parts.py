@@ -200,15 +200,6 @@ class _MatrixStateMixer(EndsMixer):
         storage, index, _ = self.caches[name]
         return storage.slots(index)
 
-    def carry(self, step, heads, dk, dv, delta):
-        """Scratch for walking long runs in pieces, sized for the engine's largest step; None for steps of short runs."""
-        ops = self.ctx.ops
-        if step.max_run < 4 * ops.gated_state_piece(dk):
-            return None
-        lim = step.limits
-        rows, seqs = max(step.rows, lim.max_tokens if lim else 0), max(step.seqs, lim.max_seqs if lim else 0)
-        return step.flat("gated_state_carry", ops.gated_state_carry_floats(rows, seqs, heads, dk, dv, delta))
-
 
 class _ConvStateMixer(_MatrixStateMixer):
     """A short convolution (silu) over some of the projected channels, then a matrix state per head with one decay per head
@@ -231,6 +222,15 @@ class _ConvStateMixer(_MatrixStateMixer):
         if not single:
             ops.short_conv_state(x, state, step, taps)
         return mixed
+
+    def carry(self, step, heads, dk, dv, delta):
+        """Scratch for walking long runs in pieces, sized for the engine's largest step; None for steps of short runs."""
+        ops = self.ctx.ops
+        if step.max_run < 4 * ops.gated_state_piece(dk):
+            return None
+        lim = step.limits
+        rows, seqs = max(step.rows, lim.max_tokens if lim else 0), max(step.seqs, lim.max_seqs if lim else 0)
+        return step.flat("gated_state_carry", ops.gated_state_carry_floats(rows, seqs, heads, dk, dv, delta))
 
 
 @MIXERS.register("gated_delta")
@@ -377,10 +377,21 @@ class LightningAttention(_MatrixStateMixer):
     def bind(self, tensors):
         super().bind(tensors)
         self.w["norm"] = (self.w["norm"] * float(self.params.get("out_factor", 1.0))).contiguous()
-        self.w["decay"] = torch.tensor(self.params["decay"], dtype=torch.float32, device=self.w["norm"].device)
+        device = self.w["norm"].device
+        self.w["decay"] = torch.tensor(self.params["decay"], dtype=torch.float32, device=device)
+        if self.ctx.ops is not None:
+            self.w["powers"] = self.ctx.ops.lightning_powers(self.params["decay"], self.ctx.ops.lightning_piece(self.d), device)
 
     def cache_needs(self):
         return {"state": StateNeed((self.nh, self.d, self.dv), torch.float32)}
+
+    def carry(self, step):
+        """Scratch for runs longer than a piece, sized for the engine's largest step."""
+        ops, lim = self.ctx.ops, step.limits
+        if step.max_run <= ops.lightning_piece(self.d):
+            return None
+        rows, seqs = max(step.rows, lim.max_tokens if lim else 0), max(step.seqs, lim.max_seqs if lim else 0)
+        return step.flat("lightning_carry", ops.lightning_carry_floats(rows, seqs, self.nh, self.d, self.dv))
 
     def flops(self, rows, attended=0):
         return super().flops(rows) + rows * self.nh * 5.0 * self.d * self.dv
@@ -390,6 +401,8 @@ class LightningAttention(_MatrixStateMixer):
         nh, d, dv = self.nh, self.d, self.dv
         q, k, v, g = (proj[:, at:] for at in (0, nh * d, 2 * nh * d, 2 * nh * d + nh * dv))
         o = step.ws("lightning_o", (step.rows, nh * dv), torch.float32)
-        ops.gated_state(q, k, v, None, None, None, o, self.state("state"), step, nh, nh, d, dv, decay=w["decay"], silu_in=True,
-                        carry=self.carry(step, nh, d, dv, False))
+        if step.max_run >= ops.LIGHTNING_MIN_RUN:      # runs of rows: products on the matrix cores, chunk by chunk
+            ops.lightning(q, k, v, w["powers"], o, self.state("state"), step, nh, d, dv, silu_in=True, carry=self.carry(step))
+        else:
+            ops.gated_state(q, k, v, None, None, None, o, self.state("state"), step, nh, nh, d, dv, decay=w["decay"], silu_in=True)
         ops.group_norm_gate(o, g, w["norm"], out, 1, nh * dv, self.params["eps"], after=True)
