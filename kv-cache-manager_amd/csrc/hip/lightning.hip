@@ -13,9 +13,10 @@
 // products alone), then the states that enter the pieces, one after another (S <- decay^piece S + part, element by element),
 // then every piece again from the state that enters it, now with outputs.  Runs of at most a piece are one launch.
 //
-// A workgroup of four waves takes one (sequence, piece, head) and a stretch of DVT value columns.  K and V of a chunk are staged
-// through LDS (the next chunk's on their way in registers meanwhile), a wave holds its 16 rows of q in registers and computes
-// their outputs; the state stays in accumulators, a quarter of the key dimension a wave, and passes through LDS once per chunk.
+// A workgroup of four waves (or eight: CS 2, two waves share a row tile and halve its columns) takes one (sequence, piece, head)
+// and a stretch of DVT value columns.  K and V of a chunk are staged through LDS (the next chunk's on their way in registers
+// meanwhile), a wave holds its 16 rows of q in registers and computes their outputs; the state stays in accumulators, a quarter of
+// the key dimension a wave, and passes through LDS once per chunk.
 // The sum over k of a 16 x 16 x 4 instruction may take k in any order: a lane group g takes the four consecutive k = 4 g .. 4 g + 3
 // of every sixteen over four instructions, so that what lies along k is read 16 bytes at a time.
 #include "common.h"
@@ -64,10 +65,10 @@ __device__ __forceinline__ float4 load4(const float* row, int i, int n, bool in)
 __device__ __forceinline__ float4 silu4(float4 x) { return float4{silu<bf16_t>(x.x), silu<bf16_t>(x.y), silu<bf16_t>(x.z), silu<bf16_t>(x.w)}; }
 
 // PARTS: the first of the three launches (no outputs; the piece's own part of the state goes to the carry)
-template <int DKP, int DVT, bool WIDE, bool PARTS>
-__global__ void __launch_bounds__(256) lightning_kernel(LightningArgs A) {
+template <int DKP, int DVT, int CS, bool WIDE, bool PARTS>
+__global__ void __launch_bounds__(256 * CS) lightning_kernel(LightningArgs A) {
   constexpr int C = kLtRows, KP = DKP + 4, VP = DVT + 4, PP = C + 4;      // pitches: rows four apart lie 16 banks apart
-  constexpr int BT = DKP / 64, CT = DVT / 16, KS = DKP / 16;
+  constexpr int BT = DKP / 64, CT = DVT / 16 / CS, KS = DKP / 16, NT = 256 * CS;
   __shared__ __attribute__((aligned(16))) float Ks[C][KP];
   __shared__ __attribute__((aligned(16))) float Vs[C][VP];
   __shared__ __attribute__((aligned(16))) float Ss[PARTS ? 1 : DKP][VP];
@@ -75,7 +76,8 @@ __global__ void __launch_bounds__(256) lightning_kernel(LightningArgs A) {
   __shared__ float pw[C + 1];
   const int head = blockIdx.x / A.col_blocks, c0 = (blockIdx.x % A.col_blocks) * DVT;
   const int s = blockIdx.y / A.pieces_per_seq, p = blockIdx.y % A.pieces_per_seq;
-  const int tid = threadIdx.x, wave = tid / kWave, lane = tid % kWave, col = lane % 16, g = lane / 16;
+  const int tid = threadIdx.x, wave = (tid / kWave) % 4, half = tid / 256, lane = tid % kWave, col = lane % 16, g = lane / 16;
+  const int cw = half * CT * 16;      // where this wave's columns of the stretch start
   const int dk = A.dk, dv = A.dv;
   const int run0 = A.run_start[s], run1 = A.run_start[s + 1], slot = A.state_slots[s];
   const bool pieces = A.piece > 0;
@@ -86,7 +88,7 @@ __global__ void __launch_bounds__(256) lightning_kernel(LightningArgs A) {
   if (PARTS && (last || slot < 0)) return;      // nothing follows the last piece
   const int cols = dv - c0 < DVT ? dv - c0 : DVT;
   if (slot < 0) {
-    for (int e = tid; e < (r1 - r0) * cols; e += 256) A.o[size_t(r0 + e / cols) * A.ldo + size_t(head) * dv + c0 + e % cols] = 0.f;
+    for (int e = tid; e < (r1 - r0) * cols; e += NT) A.o[size_t(r0 + e / cols) * A.ldo + size_t(head) * dv + c0 + e % cols] = 0.f;
     return;
   }
   if (tid <= C) pw[tid] = A.powers[size_t(head) * (C + 2) + tid];
@@ -103,22 +105,22 @@ __global__ void __launch_bounds__(256) lightning_kernel(LightningArgs A) {
       for (int ct = 0; ct < CT; ++ct)
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
-          const int key = (wave * BT + b) * 16 + g * 4 + i, c = ct * 16 + col;
+          const int key = (wave * BT + b) * 16 + g * 4 + i, c = cw + ct * 16 + col;
           S[b][ct][i] = src && key < dk && c < cols ? src[size_t(key) * dv + c0 + c] : 0.f;
         }
   }
 
-  constexpr int KQ = C * DKP / 4 / 256, VQ = C * DVT / 4 / 256;
+  constexpr int KQ = C * DKP / 4 / NT, VQ = C * DVT / 4 / NT;
   float4 kreg[KQ], vreg[VQ], qreg[PARTS ? 1 : KS];
   auto request = [&](int t0) {      // rows t0 .. t0 + 63 of the piece; what lies outside is zero
 #pragma unroll
     for (int n = 0; n < KQ; ++n) {
-      const int e = tid + n * 256, row = e / (DKP / 4), i = (e % (DKP / 4)) * 4;
+      const int e = tid + n * NT, row = e / (DKP / 4), i = (e % (DKP / 4)) * 4;
       kreg[n] = load4<WIDE>(A.k + size_t(t0 + row < r1 ? t0 + row : r1 - 1) * A.ldk + size_t(head) * dk, i, dk, t0 + row < r1);
     }
 #pragma unroll
     for (int n = 0; n < VQ; ++n) {
-      const int e = tid + n * 256, row = e / (DVT / 4), c = (e % (DVT / 4)) * 4;
+      const int e = tid + n * NT, row = e / (DVT / 4), c = (e % (DVT / 4)) * 4;
       vreg[n] = load4<WIDE>(A.v + size_t(t0 + row < r1 ? t0 + row : r1 - 1) * A.ldv + size_t(head) * dv + c0, c, cols, t0 + row < r1);
     }
     if constexpr (!PARTS) {
@@ -135,12 +137,12 @@ __global__ void __launch_bounds__(256) lightning_kernel(LightningArgs A) {
     __syncthreads();      // the chunk before is done with Ks, Vs and Ss
 #pragma unroll
     for (int m = 0; m < KQ; ++m) {
-      const int e = tid + m * 256;
+      const int e = tid + m * NT;
       *reinterpret_cast<float4*>(&Ks[e / (DKP / 4)][(e % (DKP / 4)) * 4]) = A.silu_in ? silu4(kreg[m]) : kreg[m];
     }
 #pragma unroll
     for (int m = 0; m < VQ; ++m) {
-      const int e = tid + m * 256;
+      const int e = tid + m * NT;
       *reinterpret_cast<float4*>(&Vs[e / (DVT / 4)][(e % (DVT / 4)) * 4]) = A.silu_in ? silu4(vreg[m]) : vreg[m];
     }
     float4 qf[PARTS ? 1 : KS];
@@ -152,17 +154,19 @@ __global__ void __launch_bounds__(256) lightning_kernel(LightningArgs A) {
 #pragma unroll
         for (int ct = 0; ct < CT; ++ct)
 #pragma unroll
-          for (int i = 0; i < 4; ++i) Ss[(wave * BT + b) * 16 + g * 4 + i][ct * 16 + col] = S[b][ct][i];
+          for (int i = 0; i < 4; ++i) Ss[(wave * BT + b) * 16 + g * 4 + i][cw + ct * 16 + col] = S[b][ct][i];
     }
     __syncthreads();
     if (t0 + C < r1) request(t0 + C);      // on its way while this chunk is multiplied
 
     if constexpr (!PARTS) {
-      if (wave * 16 < n) {
+      const bool busy = wave * 16 < n;
+      if (busy) {
         // Q K^T of this wave's rows with the rows up to its own, masked and decayed, to LDS as the next product's first operand
 #pragma unroll
         for (int jt = 0; jt < 4; ++jt) {
           if (jt > wave) break;
+          if (CS > 1 && jt % CS != half) continue;      // (the row tile's other wave makes these)
           f32x4 acc = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
           for (int ks = 0; ks < KS; ++ks) {
@@ -179,6 +183,9 @@ __global__ void __launch_bounds__(256) lightning_kernel(LightningArgs A) {
           }
         }
         __builtin_amdgcn_wave_barrier();
+      }
+      if constexpr (CS > 1) __syncthreads();
+      if (busy) {
         f32x4 acc[CT];
 #pragma unroll
         for (int ct = 0; ct < CT; ++ct) acc[ct] = f32x4{0.f, 0.f, 0.f, 0.f};
@@ -189,7 +196,7 @@ __global__ void __launch_bounds__(256) lightning_kernel(LightningArgs A) {
           for (int e = 0; e < 4; ++e)
 #pragma unroll
             for (int ct = 0; ct < CT; ++ct)
-              acc[ct] = __builtin_amdgcn_mfma_f32_16x16x4f32(qe[e], Ss[ks * 16 + g * 4 + e][ct * 16 + col], acc[ct], 0, 0, 0);
+              acc[ct] = __builtin_amdgcn_mfma_f32_16x16x4f32(qe[e], Ss[ks * 16 + g * 4 + e][cw + ct * 16 + col], acc[ct], 0, 0, 0);
         }
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
@@ -206,7 +213,7 @@ __global__ void __launch_bounds__(256) lightning_kernel(LightningArgs A) {
           for (int e = 0; e < 4; ++e)
 #pragma unroll
             for (int ct = 0; ct < CT; ++ct)
-              acc[ct] = __builtin_amdgcn_mfma_f32_16x16x4f32(pe[e], Vs[jt * 16 + g * 4 + e][ct * 16 + col], acc[ct], 0, 0, 0);
+              acc[ct] = __builtin_amdgcn_mfma_f32_16x16x4f32(pe[e], Vs[jt * 16 + g * 4 + e][cw + ct * 16 + col], acc[ct], 0, 0, 0);
         }
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
@@ -215,7 +222,7 @@ __global__ void __launch_bounds__(256) lightning_kernel(LightningArgs A) {
           float* dst = A.o + size_t(t0 + row) * A.ldo + size_t(head) * dv + c0;
 #pragma unroll
           for (int ct = 0; ct < CT; ++ct)
-            if (ct * 16 + col < cols) dst[ct * 16 + col] = acc[ct][i];
+            if (cw + ct * 16 + col < cols) dst[cw + ct * 16 + col] = acc[ct][i];
         }
       }
       if (t0 + C >= r1 && !last) break;      // the state that leaves this piece is another piece's business
@@ -238,7 +245,7 @@ __global__ void __launch_bounds__(256) lightning_kernel(LightningArgs A) {
         for (int b = 0; b < BT; ++b) kf[b] = Ks[j][(wave * BT + b) * 16 + col] * w;
 #pragma unroll
         for (int ct = 0; ct < CT; ++ct) {
-          const float vf = Vs[j][ct * 16 + col];
+          const float vf = Vs[j][cw + ct * 16 + col];
 #pragma unroll
           for (int b = 0; b < BT; ++b) S[b][ct] = __builtin_amdgcn_mfma_f32_16x16x4f32(kf[b], vf, S[b][ct], 0, 0, 0);
         }
@@ -252,7 +259,7 @@ __global__ void __launch_bounds__(256) lightning_kernel(LightningArgs A) {
       for (int ct = 0; ct < CT; ++ct)
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
-          const int key = (wave * BT + b) * 16 + g * 4 + i, c = ct * 16 + col;
+          const int key = (wave * BT + b) * 16 + g * 4 + i, c = cw + ct * 16 + col;
           if (key < dk && c < cols) dst[size_t(key) * dv + c0 + c] = S[b][ct][i];
         }
   }
@@ -283,15 +290,15 @@ __global__ void __launch_bounds__(256) lightning_pass_kernel(LightningArgs A) {
   }
 }
 
-template <int DKP, int DVT, bool WIDE>
+template <int DKP, int DVT, int CS, bool WIDE>
 void launch_lightning(LightningArgs A, int S, hipStream_t s) {
   A.col_blocks = (A.dv + DVT - 1) / DVT;
   const dim3 grid(A.heads * A.col_blocks, S * A.pieces_per_seq);
   if (A.piece > 0) {
-    lightning_kernel<DKP, DVT, WIDE, true><<<grid, 256, 0, s>>>(A);
+    lightning_kernel<DKP, DVT, CS, WIDE, true><<<grid, 256 * CS, 0, s>>>(A);
     lightning_pass_kernel<<<dim3((A.dk * A.dv + 255) / 256, A.heads, S), 256, 0, s>>>(A);
   }
-  lightning_kernel<DKP, DVT, WIDE, false><<<grid, 256, 0, s>>>(A);
+  lightning_kernel<DKP, DVT, CS, WIDE, false><<<grid, 256 * CS, 0, s>>>(A);
 }
 
 }  // namespace kvcm
@@ -328,14 +335,14 @@ int kvcm_lightning(const float* q, int ldq, const float* k, int ldk, const float
   KVCM_REQUIRE(static_cast<long long>(S) * A.pieces_per_seq <= 65535 && heads <= 65535, "lightning: too many sequences and pieces for one launch");
   auto aligned = [](const void* x) { return reinterpret_cast<uintptr_t>(x) % 16 == 0; };
   const bool wide = dk % 4 == 0 && dv % 4 == 0 && ldq % 4 == 0 && ldk % 4 == 0 && ldv % 4 == 0 && aligned(q) && aligned(k) && aligned(v);
-#define KVCM_LIGHTNING(DKP, DVT)                          \
-  {                                                       \
-    if (wide) launch_lightning<DKP, DVT, true>(A, S, s);  \
-    else launch_lightning<DKP, DVT, false>(A, S, s);      \
+#define KVCM_LIGHTNING(DKP, DVT, CS)                          \
+  {                                                           \
+    if (wide) launch_lightning<DKP, DVT, CS, true>(A, S, s);  \
+    else launch_lightning<DKP, DVT, CS, false>(A, S, s);      \
   }
-  if (dk <= 64) { if (dv <= 32) KVCM_LIGHTNING(64, 32) else KVCM_LIGHTNING(64, 64) }
-  else if (dk <= 128) { if (dv <= 32) KVCM_LIGHTNING(128, 32) else KVCM_LIGHTNING(128, 64) }
-  else KVCM_LIGHTNING(256, 32)      // (wider stretches of values do not fit the local memory beside keys of this size)
+  if (dk <= 64) { if (dv <= 32) KVCM_LIGHTNING(64, 32, 1) else KVCM_LIGHTNING(64, 64, 2) }
+  else if (dk <= 128) { if (dv <= 32) KVCM_LIGHTNING(128, 32, 1) else if (dv <= 64) KVCM_LIGHTNING(128, 64, 2) else KVCM_LIGHTNING(128, 128, 2) }
+  else KVCM_LIGHTNING(256, 32, 1)      // (wider stretches of values do not fit the local memory beside keys of this size)
 #undef KVCM_LIGHTNING
   return launch_status("lightning");
 }

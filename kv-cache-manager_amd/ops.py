@@ -1885,7 +1885,9 @@ LIGHTNING_MIN_RUN = 16       # rows of a run from which its matrix form is worth
 
 
 def lightning_piece(dk):
-    """Rows of a piece when long runs are walked in pieces."""
+    """Rows of a piece when long runs are walked in pieces.  Measured on 2,048 rows of 32 heads (the three launches together):
+    64 x 64 states 54 / 51 / 59 us with pieces of 64 / 128 / 256 rows, 128 x 128 states 151 / 140 / 137 us (walked row by row in
+    pieces of their own: 111 and 260 us)."""
     return 128 if dk <= 64 else 256
 
 
